@@ -49,6 +49,7 @@ class KVGroupSpec:
     window: int = 0            # 0: all keys are kept; w > 0: the last w keys
     v_head_dim: int = 0        # size of a value where it is not that of a key
     keeps_all: bool = False    # with a window: no ring, every key stays where it was written
+    keep_first: int = 0        # with both: the first tokens that every query sees beside its window
 
     @property
     def value_dim(self) -> int:

@@ -127,6 +127,11 @@ typedef struct {
     int32_t mask_window;
     int32_t mask_chunk;
     int32_t out_float;
+    int32_t keep_first;      // the sequence's first keys that a query sees beside its window (what the decode step's work list covers)
+    float softcap;           // > 0: a scaled score s becomes softcap tanh(s / softcap); no bias by distance then
+    int32_t gate_per_head;   // 1: gate rows hold one number a head
+    int32_t out_stride;      // > 0: elements from one output row to the next (0: H dv), and the outputs are
+    float out_mult;          // multiplied by out_mult
 } picolm_attn_extras;
 // picolm_attn_prefill_generic / picolm_attn_decode_generic over pages kept as plain arrays K[64][d],
 // V^T[dv][64] whatever the dtype and head size, with the extras above; out rows are [H][dv] and the

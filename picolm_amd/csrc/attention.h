@@ -61,6 +61,15 @@ struct AttnArgs {
     int mask_chunk;
     // the output rows are float whatever the dtype of q and of the pages
     int out_float;
+    // a query sees the first `keep_first` keys of its sequence too, however far behind its window they lie
+    int keep_first;
+    // > 0: a scaled score s becomes softcap tanh(s / softcap)
+    float softcap;
+    // the gate is one number a head: gate[token * gate_stride + head]
+    int gate_per_head;
+    // > 0: elements from one output row to the next where it is not H dv, and a factor on the output
+    int out_stride;
+    float out_mult;
 };
 
 // how many keys back a query sees (0: all)
@@ -72,6 +81,12 @@ __device__ __forceinline__ int first_seen(const AttnArgs& a, int qpos) {
     if (a.mask_chunk > 0) lo = max(lo, qpos / a.mask_chunk * a.mask_chunk);
     return lo;
 }
+
+// Pages (or tiles of keys) that a query visits: `kept` of them from the sequence's start, then those
+// from `first` on.  They are counted from first - kept, so that the count of a page from `first` on is
+// its own number; what a count below `first` stands for:
+__device__ __forceinline__ int counted_page(int n, int first, int kept) { return n >= first ? n : n - (first - kept); }
+__device__ __forceinline__ float softcapped(float s, float cap) { return cap * tanhf(s / cap); }
 
 // ---- the order of a page's elements ---------------------------------------------------------
 // A page holds, per KV group, the keys K[64][d] and the values transposed V^T[d][64].  Pages of
@@ -116,12 +131,14 @@ __host__ __device__ __forceinline__ int v_page_offset(int i, int key, int d, boo
 // combines them.  The host's work list is built from the same arithmetic.  In a decode step row
 // i of q and of the output belongs to sequence i.
 struct DecodeWork {
-    int seq, split, qpos, slot, page_lo, page_hi, n_chunks;
+    int seq, split, qpos, slot, page_lo, page_hi, n_chunks;     // pages page_lo .. page_hi - 1 as counted_page counts them
+    int first_page, kept_pages;
     int phys[4];
 };
 __device__ __forceinline__ int decode_first_page(int window, int qpos) {
     return (window > 0 ? max(0, qpos - window + 1) : 0) / 64;
 }
+__device__ __forceinline__ int decode_kept_pages(int keep_first, int first_page) { return min((keep_first + 63) / 64, first_page); }
 // The decode grid is one-dimensional: workgroup b takes entry b / per_entry and is number
 // b % per_entry (KV group, chunk of heads) of that entry's workgroups, so that all workgroups of
 // entries in use are handed out before those that find nothing to do.
@@ -142,7 +159,10 @@ __device__ __forceinline__ bool decode_work(const AttnArgs& a, int per_entry, De
     w.phys[1] = e1.y;
     w.phys[2] = e1.z;
     w.phys[3] = e1.w;
-    const int first = decode_first_page(a.window, w.qpos), end = w.qpos / 64 + 1;
+    const int end = w.qpos / 64 + 1;
+    w.first_page = decode_first_page(a.window, w.qpos);
+    w.kept_pages = decode_kept_pages(a.keep_first, w.first_page);
+    const int first = w.first_page - w.kept_pages;
     w.n_chunks = (end - first + a.pages_per_chunk - 1) / a.pages_per_chunk;
     w.page_lo = first + w.split * a.pages_per_chunk;
     w.page_hi = min(end, w.page_lo + a.pages_per_chunk);

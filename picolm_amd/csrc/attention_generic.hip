@@ -75,9 +75,12 @@ __global__ __launch_bounds__(AT_THREADS) void attn_tile_kernel(AttnArgs a) {
     const int qpos_first = row_qpos[0], qpos_last = row_qpos[n_rows - 1];
     const int hi = qpos_last;
     const int lo = row_lo[0];                                         // (the tile's first query sees furthest back)
-    int page_lo = lo / PAGE_TOKENS, page_hi = hi / PAGE_TOKENS + 1;   // [page_lo, page_hi)
+    const int seen_lo = lo / PAGE_TOKENS;
+    int first_page = seen_lo, kept = min((a.keep_first + PAGE_TOKENS - 1) / PAGE_TOKENS, first_page);
+    int page_lo = first_page - kept, page_hi = hi / PAGE_TOKENS + 1;   // [page_lo, page_hi) as counted_page counts them
     if (a.decode) {
-        page_lo = max(work.page_lo, page_lo);
+        first_page = work.first_page, kept = work.kept_pages;
+        page_lo = kept > 0 ? work.page_lo : max(work.page_lo, seen_lo);
         page_hi = work.page_hi;
     }
 
@@ -108,7 +111,8 @@ __global__ __launch_bounds__(AT_THREADS) void attn_tile_kernel(AttnArgs a) {
     const int32_t* pt = a.page_table + (size_t)slot * a.max_pages;
     const size_t page_elems = (size_t)a.G * PAGE_TOKENS * d, v_page_elems = (size_t)a.G * PAGE_TOKENS * dv;
 
-    for (int page = page_lo; page < page_hi; ++page) {
+    for (int counted = page_lo; counted < page_hi; ++counted) {
+        const int page = counted_page(counted, first_page, kept);
         const int phys = pt[page % a.ring_pages];
         const size_t base = (size_t)phys * page_elems + (size_t)g * PAGE_TOKENS * d;
         const size_t v_base = (size_t)phys * v_page_elems + (size_t)g * PAGE_TOKENS * dv;
@@ -140,10 +144,11 @@ __global__ __launch_bounds__(AT_THREADS) void attn_tile_kernel(AttnArgs a) {
             for (int i = 0; i < 4; ++i) {
                 const int r = 4 * wave + i;
                 const int qp = row_qpos[r];
-                const bool vis = r < n_rows && kpos <= qp && kpos >= row_lo[r];
+                const bool vis = r < n_rows && kpos <= qp && (kpos >= row_lo[r] || kpos < a.keep_first);
                 float sc = NEG_BIG;
                 if (vis) {
                     sc = s[i] * a.scale;
+                    if (a.softcap > 0.f) sc = softcapped(sc, a.softcap);
                     if (a.bias) sc += a.bias[(size_t)row_head[r] * a.bias_rows + min(qp - kpos, a.bias_rows - 1)];
                 }
                 const float m_new = fmaxf(m_run[i], wave_max(sc));
@@ -209,13 +214,14 @@ __global__ __launch_bounds__(AT_THREADS) void attn_tile_kernel(AttnArgs a) {
             l = l * keep + expf(a.sink[head] - top);
         }
         const float inv = l > 0.f ? keep / l : 0.f;
-        const size_t at = (size_t)tok * a.H * dv + (size_t)head * dv;
-        const float* gate = a.gate ? a.gate + (size_t)tok * a.gate_stride + (size_t)head * dv : nullptr;
+        const size_t at = (size_t)tok * (a.out_stride ? a.out_stride : a.H * dv) + (size_t)head * dv;
+        const float* gate = a.gate ? a.gate + (size_t)tok * a.gate_stride + (size_t)head * (a.gate_per_head ? 1 : dv) : nullptr;
+        const float mult = a.out_stride ? a.out_mult : 1.f;
 #pragma unroll
         for (int j = 0; j < MAXD / 16; ++j)
             if (j < n_cg) {
-                float y = acc[j] * inv;
-                if (gate) y *= 1.f / (1.f + expf(-gate[pc + 16 * j]));
+                float y = acc[j] * inv * mult;
+                if (gate) y *= 1.f / (1.f + expf(-gate[a.gate_per_head ? 0 : pc + 16 * j]));
                 if (a.out_float) ((float*)a.out)[at + pc + 16 * j] = y;
                 else ((T*)a.out)[at + pc + 16 * j] = from_f32<T>(y);
             }
@@ -233,7 +239,8 @@ __global__ __launch_bounds__(MERGE_WAVES * WAVE) void attn_merge_kernel(AttnArgs
     const int H = a.H, d = a.dv > 0 ? a.dv : a.d;        // columns of a value
     const int seq = unit / H, head = unit % H;
     const int qpos = a.seq_pos0[seq];
-    const int n_splits = (qpos / 64 + 1 - decode_first_page(a.window, qpos) + a.pages_per_chunk - 1) / a.pages_per_chunk;
+    const int first_page = decode_first_page(a.window, qpos), kept = decode_kept_pages(a.keep_first, first_page);
+    const int n_splits = (qpos / 64 + 1 - first_page + kept + a.pages_per_chunk - 1) / a.pages_per_chunk;
     if (n_splits <= 1) return;                         // its one workgroup wrote the result itself
     const int stride = d + 2;
     const float* p = a.partial + (size_t)unit * a.max_splits * stride;
@@ -256,13 +263,14 @@ __global__ __launch_bounds__(MERGE_WAVES * WAVE) void attn_merge_kernel(AttnArgs
     for (int i = lane; i < n_splits; i += WAVE) l += expf(p[(size_t)i * stride] - M) * p[(size_t)i * stride + 1];
     float L = wave_sum(l);
     if (a.sink) L += expf(a.sink[head] - M);
-    const float inv = L > 0.f ? 1.0f / L : 0.f;
-    const size_t at = (size_t)seq * H * d + (size_t)head * d;
+    const float inv = (L > 0.f ? 1.0f / L : 0.f) * (a.out_stride ? a.out_mult : 1.f);
+    const size_t at = (size_t)seq * (a.out_stride ? a.out_stride : H * d) + (size_t)head * d;
     auto store = [&](int c, float y) {
         if (a.out_float) ((float*)a.out)[at + c] = y;
         else ((T*)a.out)[at + c] = from_f32<T>(y);
     };
-    const float* gate = a.gate ? a.gate + (size_t)seq * a.gate_stride + (size_t)head * d : nullptr;
+    const float* gate = a.gate ? a.gate + (size_t)seq * a.gate_stride + (size_t)head * (a.gate_per_head ? 1 : d) : nullptr;
+    const auto gate_at = [&](int c) { return gate[a.gate_per_head ? 0 : c]; };
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
         const int c = lane + j * WAVE;
@@ -272,13 +280,13 @@ __global__ __launch_bounds__(MERGE_WAVES * WAVE) void attn_merge_kernel(AttnArgs
         for (int i = 0; i < EARLY; ++i)
             if (i < n_splits) acc += expf(p[(size_t)i * stride] - M) * early[i][j];
         for (int i = EARLY; i < n_splits; ++i) acc += expf(p[(size_t)i * stride] - M) * p[(size_t)i * stride + 2 + c];
-        if (gate) acc *= 1.f / (1.f + expf(-gate[c]));
+        if (gate) acc *= 1.f / (1.f + expf(-gate_at(c)));
         store(c, acc * inv);
     }
     for (int c = lane + 4 * WAVE; c < d; c += WAVE) {       // a head wider than 256
         float acc = 0.f;
         for (int i = 0; i < n_splits; ++i) acc += expf(p[(size_t)i * stride] - M) * p[(size_t)i * stride + 2 + c];
-        if (gate) acc *= 1.f / (1.f + expf(-gate[c]));
+        if (gate) acc *= 1.f / (1.f + expf(-gate_at(c)));
         store(c, acc * inv);
     }
 }
@@ -397,6 +405,8 @@ static void with_extras(AttnArgs& a, const picolm_attn_extras* x) {
     a.mask_window = x->mask_window;
     a.mask_chunk = x->mask_chunk;
     a.out_float = x->out_float;
+    a.keep_first = x->keep_first, a.softcap = x->softcap, a.gate_per_head = x->gate_per_head;
+    a.out_stride = x->out_stride, a.out_mult = x->out_mult;
 }
 
 static int check_extras(const char* who, const picolm_attn_extras* x, int H, int d) {
@@ -404,7 +414,10 @@ static int check_extras(const char* who, const picolm_attn_extras* x, int H, int
     PICOLM_REQUIRE(x->v_head_dim >= 0 && x->v_head_dim <= AT_MAX_D, "%s: value size %d is not in [1, %d]", who, x->v_head_dim, AT_MAX_D);
     PICOLM_REQUIRE(!x->bias || x->bias_rows >= 1, "%s: a bias by distance needs at least one row", who);
     const int dv = x->v_head_dim > 0 ? x->v_head_dim : d;
-    PICOLM_REQUIRE(!x->gate || x->gate_stride >= H * dv, "%s: gate rows of %d floats for %d heads of %d", who, x->gate_stride, H, dv);
+    PICOLM_REQUIRE(!x->gate || x->gate_stride >= (x->gate_per_head ? H : H * dv), "%s: gate rows of %d floats for %d heads of %d", who, x->gate_stride, H, dv);
+    PICOLM_REQUIRE(x->keep_first >= 0 && x->softcap >= 0.f && !(x->bias && x->softcap > 0.f) && (!x->out_stride || x->out_stride >= H * dv),
+                   "%s: %d kept keys, a cap of %g (which takes no bias by distance), output rows of %d for %d heads of %d", who, x->keep_first,
+                   (double)x->softcap, x->out_stride, H, dv);
     PICOLM_REQUIRE(x->mask_window >= 0, "%s: a window of %d keys", who, x->mask_window);
     PICOLM_REQUIRE(x->mask_chunk >= 0, "%s: stretches of %d keys", who, x->mask_chunk);
     return 0;

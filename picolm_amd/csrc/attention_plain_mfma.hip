@@ -61,7 +61,7 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
     extern __shared__ float merge_lds[];        // [PLAIN_WAVES - 1][DV / 2 + 2][64]: O^T, maximum and sum of the other waves
     const int lane = threadIdx.x % 64, wave = threadIdx.x / 64, col = lane & 31, h = lane >> 5;
     const int R = a.H / a.G;
-    int seq, g, head, tok, qpos, qpos_first, slot, page_lo, page_hi, hi, split = 0, n_chunks = 1;
+    int seq, g, head, tok, qpos, qpos_first, slot, page_lo, page_hi, hi, split = 0, n_chunks = 1, first_tile, kept_tiles;
     bool q_ok;
     if (a.decode) {
         DecodeWork w;
@@ -75,6 +75,7 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
         head = g * R + min(j, R - 1);
         tok = seq, qpos = qpos_first = w.qpos, hi = w.qpos;
         page_lo = w.page_lo, page_hi = w.page_hi;
+        first_tile = 2 * w.first_page, kept_tiles = 2 * w.kept_pages;
     } else {
         seq = a.tile_seq[blockIdx.x];
         const int q0 = a.tile_q0[blockIdx.x], nnew = a.seq_nnew[seq], pos0 = a.seq_pos0[seq];
@@ -85,7 +86,9 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
         tok = a.cu_seqlens[seq] + l, qpos = pos0 + l, qpos_first = pos0 + q0;
         slot = a.seq_slot[seq];
         hi = pos0 + min(q0 + 31, nnew - 1);
-        page_lo = first_seen(a, qpos_first) / PAGE_TOKENS, page_hi = hi / PAGE_TOKENS + 1;      // (the tile's first query sees furthest back)
+        first_tile = first_seen(a, qpos_first) / 32;      // (the tile's first query sees furthest back)
+        kept_tiles = min((a.keep_first + 31) / 32, first_tile);
+        page_lo = first_tile / 2, page_hi = hi / PAGE_TOKENS + 1;
     }
     // the wave's queries as operands: column `col`, k-step s covers elements 16 s + 8 h .. + 8
     bf16x8 Qf[D / 16];
@@ -101,6 +104,7 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
         for (int e = 0; e < 16; ++e) O[dt][e] = 0.f;
     float m_run = NEG_BIG, l_run = 0.f;
     const float scale2 = a.scale * LOG2E;
+    const float cap2 = a.softcap * LOG2E, scale_cap = a.softcap > 0.f ? 2.f * scale2 / a.softcap : 0.f;
     const float* bias = a.bias ? a.bias + (size_t)head * a.bias_rows : nullptr;
     const int last_row = a.bias_rows - 1;
     // (qpos_first is the wave's query nearest to the keys: a tile beyond the table's reach from there has one bias)
@@ -113,21 +117,23 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
     const int tile_hi = min(2 * page_hi, hi / 32 + 1);       // tiles of 32 keys: this wave takes tile_lo, tile_lo + PLAIN_WAVES, ... below tile_hi
     const bool keys_in_turn = !a.waves_take_heads;           // the waves share one head's keys
     const int tile_step = keys_in_turn ? PLAIN_WAVES : 1;
-    // with a window or stretches, the tile of 32 keys that holds the oldest key any query of this wave sees
+    // with a window or stretches, the tile of 32 keys that holds the oldest key any query of this wave sees; kept first
+    // tokens: their tiles come ahead of those (tiles are counted as counted_page counts, from first_tile - kept_tiles on)
     const int oldest = first_seen(a, qpos_first), my_oldest = first_seen(a, qpos);
-    const int tile_lo = max(2 * page_lo, oldest / 32) + (keys_in_turn ? wave : 0);
+    const int tile_lo = (kept_tiles == 0 ? max(2 * page_lo, oldest / 32) : a.decode ? 2 * page_lo : first_tile - kept_tiles) + (keys_in_turn ? wave : 0);
     // two sets of operands in turn: the loads of the tile after this one are queued before this
     // tile's products and stay there (the scheduler may not move them past the barrier), and the
     // page of the tile after that is looked up meanwhile
     TileOperands<D, DV> A, B;
-    auto fetch = [&](TileOperands<D, DV>& ops, int t, int phys) {
+    auto fetch = [&](TileOperands<D, DV>& ops, int counted, int phys) {
+        const int t = counted_page(counted, first_tile, kept_tiles);
         load_tile<D, DV>(ops, kbase + (size_t)phys * k_page_elems, vbase + (size_t)phys * v_page_elems, t & 1, lane);
     };
-    auto page_of = [&](int t) { return t < tile_hi ? pt[(t / 2) % a.ring_pages] : 0; };
+    auto page_of = [&](int t) { return t < tile_hi ? pt[(counted_page(t, first_tile, kept_tiles) / 2) % a.ring_pages] : 0; };
     // a tile's 16 biases of a lane, in base-2 units: asked for before the next tile's operands, because
     // loads come back in the order they were queued and the softmax must not wait for those too
     auto load_bias = [&](int t, float (&bv)[16]) {
-        const int key0 = 32 * t;
+        const int key0 = 32 * counted_page(t, first_tile, kept_tiles);
         if (!bias || t >= tile_hi) {
 #pragma unroll
             for (int e = 0; e < 16; ++e) bv[e] = 0.f;
@@ -141,18 +147,25 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
         }
     };
     auto attend = [&](const TileOperands<D, DV>& ops, int t, const float (&bv)[16]) {
-        const int key0 = 32 * t;
+        const int key0 = 32 * counted_page(t, first_tile, kept_tiles);
         f32x16 S;
 #pragma unroll
         for (int e = 0; e < 16; ++e) S[e] = 0.f;
 #pragma unroll
         for (int s = 0; s < D / 16; ++s) S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ops.K[s], Qf[s], S, 0, 0, 0);
         float mx = NEG_BIG;
+        if (a.softcap > 0.f) {          // cap tanh(s / cap) in base-2 units: cap log2(e) (1 - 2 / (1 + e^(2 s / cap)))
+#pragma unroll
+            for (int e = 0; e < 16; ++e) S[e] = cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(1.f + exp2_flushing(S[e] * scale_cap));
+        } else {
+#pragma unroll
+            for (int e = 0; e < 16; ++e) S[e] = fmaf(S[e], scale2, bv[e]);
+        }
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
             const int key = key0 + key_of_elem(e, h);
-            const bool vis = q_ok && key <= qpos && key >= my_oldest;
-            S[e] = vis ? fmaf(S[e], scale2, bv[e]) : NEG_BIG;
+            const bool vis = q_ok && key <= qpos && (key >= my_oldest || key < a.keep_first);
+            S[e] = vis ? S[e] : NEG_BIG;
             mx = fmaxf(mx, S[e]);
         }
         mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
@@ -244,9 +257,14 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
         keep = exp2_flushing(m_run - top);
         l_run = l_run * keep + exp2_flushing(s2 - top);
     }
-    const float inv = l_run > 0.f ? keep / l_run : 0.f;
-    const size_t at = (size_t)tok * a.H * DV + (size_t)head * DV;
-    const float* gate = a.gate ? a.gate + (size_t)tok * a.gate_stride + (size_t)head * DV : nullptr;
+    float inv = l_run > 0.f ? keep / l_run : 0.f;
+    if (a.out_stride) inv *= a.out_mult;
+    const size_t at = (size_t)tok * (a.out_stride ? a.out_stride : a.H * DV) + (size_t)head * DV;
+    const float* gate = a.gate ? a.gate + (size_t)tok * a.gate_stride + (size_t)head * (a.gate_per_head ? 1 : DV) : nullptr;
+    if (gate && a.gate_per_head) {
+        inv *= 1.f / (1.f + __expf(-gate[0]));
+        gate = nullptr;
+    }
 #pragma unroll
     for (int dt = 0; dt < DV / 32; ++dt)
 #pragma unroll
@@ -287,13 +305,19 @@ static int fill_extras(const char* who, AttnArgs& a, const picolm_attn_extras* x
     a.dv = dv == a.d ? 0 : dv;
     if (!x) return 0;
     PICOLM_REQUIRE(!x->bias || x->bias_rows >= 1, "%s: a bias by distance needs at least one row", who);
-    PICOLM_REQUIRE(!x->gate || x->gate_stride >= a.H * dv, "%s: gate rows of %d floats for %d heads of %d", who, x->gate_stride, a.H, dv);
+    PICOLM_REQUIRE(!x->gate || x->gate_stride >= (x->gate_per_head ? a.H : a.H * dv), "%s: gate rows of %d floats for %d heads of %d", who,
+                   x->gate_stride, a.H, dv);
+    PICOLM_REQUIRE(x->keep_first >= 0 && x->softcap >= 0.f && !(x->bias && x->softcap > 0.f) && (!x->out_stride || x->out_stride >= a.H * dv),
+                   "%s: %d kept keys, a cap of %g (which takes no bias by distance), output rows of %d for %d heads of %d", who, x->keep_first,
+                   (double)x->softcap, x->out_stride, a.H, dv);
     PICOLM_REQUIRE(x->mask_window >= 0 && (a.window <= 0 || x->mask_window <= a.window), "%s: a window of %d keys over pages laid out for %d", who,
                    x->mask_window, a.window);
     a.bias = x->bias, a.bias_rows = x->bias_rows, a.sink = x->sink, a.gate = x->gate, a.gate_stride = x->gate_stride;
     a.mask_window = x->mask_window;
     PICOLM_REQUIRE(x->mask_chunk >= 0, "%s: stretches of %d keys", who, x->mask_chunk);
     a.mask_chunk = x->mask_chunk, a.out_float = x->out_float;
+    a.keep_first = x->keep_first, a.softcap = x->softcap, a.gate_per_head = x->gate_per_head;
+    a.out_stride = x->out_stride, a.out_mult = x->out_mult;
     return 0;
 }
 

@@ -18,6 +18,7 @@
 #define VIEW_REQUIRE(who, v)                                                                                      \
     PICOLM_REQUIRE((v) && (v)->struct_bytes == (int32_t)sizeof(picolm_step_view), "%s: the step view is of another version", who)
 
+__device__ __forceinline__ float silu_f(float x) { return x / (1.f + expf(-x)); }
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
 // e^x for x <= 0 through the hardware's 2^y, with the rounding of y = x log2(e) carried along:
@@ -47,7 +48,8 @@ struct DecayScan {
     const int32_t* seq_slot;
     int64_t slot_floats;
     int qk_stride, q_off, k_off, a_off, x_stride, x_off, dt_stride, dt_off;
-    int kind, heads, key_heads, key_dim, value_dim;
+    int kind, heads, key_heads, key_dim, value_dim, act;
+    float q_scale, k_scale;
     int R, kpt, n_waves, n_cb;
     int mode, chunk_len, chunks_per_seq;      // mode 0: whole sequences; 1: (N, P) of every chunk; 3: outputs from the chunks' start states
     float* ws;                                // [sequence][chunk][head][N | P | S_start][key_dim][value_dim]
@@ -57,7 +59,7 @@ __device__ __forceinline__ float* ds_ws(const DecayScan& a, int seq, int chunk, 
     return a.ws + ((((size_t)seq * a.chunks_per_seq + chunk) * a.heads + head) * 3 + part) * a.key_dim * a.value_dim;
 }
 
-// KIND: 1 a decay per row, 2 exp(dt A) per element; TRACK: pass 1 of the chunked walk (no outputs, the decays' products kept)
+// KIND: 1 a decay per row, 2 exp(dt A) per element, 3 a fixed decay per head; TRACK: pass 1 of the chunked walk (no outputs, the decays' products kept)
 template <int R, int KIND, bool TRACK>
 __global__ __launch_bounds__(256) void decay_scan_kernel(DecayScan a) {
     extern __shared__ float ds_lds[];
@@ -95,6 +97,8 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(DecayScan a) {
         Ar[i] = in && KIND == 2 ? a.A[channel * a.key_dim + kr] : 0.f;
     }
     const float skip = a.skip && valid ? a.skip[channel] : 0.f;
+    const float fixed = KIND == 3 ? a.A[head] : 0.f;
+    const auto read = [&](float y) { return a.act ? silu_f(y) : y; };
     for (int b0 = row0; b0 < row1; b0 += DS_TB) {
         const int nb = min(DS_TB, row1 - b0);
         __syncthreads();
@@ -102,15 +106,17 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(DecayScan a) {
             const int t = idx / kd, i = idx % kd;
             const float* src = a.qk + (size_t)(b0 + t) * a.qk_stride + (size_t)kh * a.key_dim + i;
             const bool in = i < a.key_dim;
-            ks[idx] = in ? src[a.k_off] : 0.f;
-            qs[idx] = in ? src[a.q_off] : 0.f;
-            if (KIND == 1) as[idx] = in ? src[a.a_off] : 0.f;
+            ks[idx] = in ? read(src[a.k_off]) * a.k_scale : 0.f;
+            if (!TRACK) qs[idx] = in ? read(src[a.q_off]) * a.q_scale : 0.f;
+            if (KIND == 1)
+                as[idx] = !in ? 0.f
+                          : a.dt_stride > 0 ? a.dt[(size_t)(b0 + t) * a.dt_stride + a.dt_off + (size_t)kh * a.key_dim + i] : src[a.a_off];
         }
         for (int idx = tid; idx < nb * CB; idx += blockDim.x) {
             const int t = idx / CB, c = cb * CB + idx % CB;
             const bool in = c < a.value_dim;
             const size_t ch = (size_t)head * a.value_dim + c;
-            xs[idx] = in ? a.x[(size_t)(b0 + t) * a.x_stride + a.x_off + ch] : 0.f;
+            xs[idx] = in ? read(a.x[(size_t)(b0 + t) * a.x_stride + a.x_off + ch]) : 0.f;
             if (KIND == 2)
                 dts[idx] = in ? softplus_f(a.dt[(size_t)(b0 + t) * a.dt_stride + a.dt_off + ch] + (a.dt_bias ? a.dt_bias[ch] : 0.f)) : 0.f;
         }
@@ -125,10 +131,11 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(DecayScan a) {
             float o = 0.f;
 #pragma unroll
             for (int i = 0; i < DS_KPT; ++i) {
-                const float decay = KIND == 2 ? exp_of_decay(dtv * Ar[i]) : ar[i * R];
+                const float decay = KIND == 2 ? exp_of_decay(dtv * Ar[i]) : KIND == 3 ? fixed : ar[i * R];
                 S[i] = decay * S[i] + k[i * R] * wv;
-                if (TRACK) P[i] *= decay;
-                else o += S[i] * q[i * R];
+                if (TRACK && KIND != 3) P[i] *= decay;
+                if (TRACK) continue;
+                o += S[i] * q[i * R];
             }
             if (TRACK) continue;
             for (int off = CW; off < WAVE; off <<= 1) o += __shfl_xor(o, off, WAVE);
@@ -137,7 +144,7 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(DecayScan a) {
     }
     if (a.mode == 3) return;
     float* n_out = a.mode == 0 ? st : ds_ws(a, seq, chunk, head, 0);
-    float* p_out = TRACK ? ds_ws(a, seq, chunk, head, 1) : nullptr;
+    float* p_out = TRACK && KIND != 3 ? ds_ws(a, seq, chunk, head, 1) : nullptr;
 #pragma unroll
     for (int i = 0; i < DS_KPT; ++i) {
         const int kr = i * R + r;
@@ -161,9 +168,19 @@ __global__ void decay_carry_kernel(DecayScan a) {
     const int n_chunks = (n + a.chunk_len - 1) / a.chunk_len;
     float* st = a.state + (size_t)a.seq_slot[seq] * a.slot_floats + (size_t)e;
     float s = *st;
+    float whole = 1.f, rest = 1.f;      // a fixed decay over a whole chunk, and over the last one
+    if (a.kind == 3) {
+        const float decay = a.A[head];
+        const int n_rest = n - (n_chunks - 1) * a.chunk_len;
+        for (int t = 0; t < a.chunk_len; ++t) {
+            whole *= decay;
+            if (t < n_rest) rest *= decay;
+        }
+    }
     for (int c = 0; c < n_chunks; ++c) {
         ds_ws(a, seq, c, head, 2)[within] = s;
-        s = ds_ws(a, seq, c, head, 1)[within] * s + ds_ws(a, seq, c, head, 0)[within];
+        const float decay = a.kind == 3 ? (c + 1 < n_chunks ? whole : rest) : ds_ws(a, seq, c, head, 1)[within];
+        s = decay * s + ds_ws(a, seq, c, head, 0)[within];
     }
     *st = s;
 }
@@ -192,11 +209,11 @@ extern "C" int picolm_call_decay_scan(void* user, const picolm_step_view* v) {
     VIEW_REQUIRE("decay_scan", v);
     PICOLM_REQUIRE(a && v->in && v->out && v->extra[0] && v->state, "decay_scan: buffers or state are missing");
     const int heads = a->n_heads, kh = a->n_key_heads, kd = a->key_dim, vd = a->value_dim;
-    PICOLM_REQUIRE((a->kind == 1 || a->kind == 2) && heads > 0 && kh > 0 && heads % kh == 0 && kd > 0 && kd <= DS_MAX_KEY_DIM && vd > 0,
+    PICOLM_REQUIRE(a->kind >= 1 && a->kind <= 3 && heads > 0 && kh > 0 && heads % kh == 0 && kd > 0 && kd <= DS_MAX_KEY_DIM && vd > 0,
                    "decay_scan: kind %d, %d heads over %d, keys of %d (up to %d), values of %d", a->kind, heads, kh, kd, DS_MAX_KEY_DIM, vd);
     const int64_t channels = (int64_t)heads * vd;
     PICOLM_REQUIRE(a->q_off >= 0 && a->q_off + kh * kd <= a->qk_stride && a->k_off >= 0 && a->k_off + kh * kd <= a->qk_stride &&
-                       (a->kind != 1 || (a->a_off >= 0 && a->a_off + kh * kd <= a->qk_stride)) && v->extra_row_bytes[0] >= a->qk_stride * 4,
+                       (a->kind != 1 || a->dt_stride > 0 || (a->a_off >= 0 && a->a_off + kh * kd <= a->qk_stride)) && v->extra_row_bytes[0] >= a->qk_stride * 4,
                    "decay_scan: the rows of %d floats do not hold q, k and the decays at the offsets named", a->qk_stride);
     PICOLM_REQUIRE(a->x_off >= 0 && a->x_off + channels <= a->x_stride && v->in_row_bytes >= (int64_t)a->x_stride * 4 &&
                        v->out_row_bytes >= channels * 4,
@@ -204,6 +221,11 @@ extern "C" int picolm_call_decay_scan(void* user, const picolm_step_view* v) {
     PICOLM_REQUIRE(a->kind != 2 || (a->A && v->extra[1] && a->dt_off >= 0 && a->dt_off + channels <= a->dt_stride &&
                                     v->extra_row_bytes[1] >= (int64_t)a->dt_stride * 4),
                    "decay_scan: decays of the exponential kind need A and a step size per channel");
+    PICOLM_REQUIRE(a->kind != 1 || a->dt_stride <= 0 || (v->extra[1] && a->dt_off >= 0 && a->dt_off + kh * kd <= a->dt_stride &&
+                                                         v->extra_row_bytes[1] >= (int64_t)a->dt_stride * 4),
+                   "decay_scan: the decays' rows of %d floats do not hold %d at %d", a->dt_stride, kh * kd, a->dt_off);
+    PICOLM_REQUIRE(a->kind != 3 || a->A, "decay_scan: fixed decays are missing");
+    PICOLM_REQUIRE(a->act == 0 || a->act == 1, "decay_scan: unknown activation %d", a->act);
     const int64_t need = (a->state_off + channels * kd) * 4;
     PICOLM_REQUIRE(a->state_off >= 0 && need <= v->state_bytes_per_slot, "decay_scan: the state of a slot has %lld bytes, the matrices need %lld",
                    (long long)v->state_bytes_per_slot, (long long)need);
@@ -219,6 +241,7 @@ extern "C" int picolm_call_decay_scan(void* user, const picolm_step_view* v) {
     s.slot_floats = v->state_bytes_per_slot / 4;
     s.qk_stride = a->qk_stride, s.q_off = a->q_off, s.k_off = a->k_off, s.a_off = a->a_off;
     s.x_stride = a->x_stride, s.x_off = a->x_off, s.dt_stride = a->dt_stride, s.dt_off = a->dt_off;
+    s.act = a->act, s.q_scale = a->q_scale != 0.f ? a->q_scale : 1.f, s.k_scale = a->k_scale != 0.f ? a->k_scale : 1.f;
     s.kind = a->kind, s.heads = heads, s.key_heads = kh, s.key_dim = kd, s.value_dim = vd;
     int R = 1;
     while (R * DS_KPT < kd) R *= 2;
@@ -240,6 +263,8 @@ extern "C" int picolm_call_decay_scan(void* user, const picolm_step_view* v) {
     do {                                                                                                          \
         if (s.kind == 1 && s.mode == 1) decay_scan_kernel<RR, 1, true><<<grid, block, lds, v->stream>>>(s);       \
         else if (s.kind == 1) decay_scan_kernel<RR, 1, false><<<grid, block, lds, v->stream>>>(s);                \
+        else if (s.kind == 3 && s.mode == 1) decay_scan_kernel<RR, 3, true><<<grid, block, lds, v->stream>>>(s);  \
+        else if (s.kind == 3) decay_scan_kernel<RR, 3, false><<<grid, block, lds, v->stream>>>(s);                \
         else if (s.mode == 1) decay_scan_kernel<RR, 2, true><<<grid, block, lds, v->stream>>>(s);                 \
         else decay_scan_kernel<RR, 2, false><<<grid, block, lds, v->stream>>>(s);                                 \
     } while (0)

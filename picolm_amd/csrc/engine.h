@@ -72,6 +72,7 @@ typedef struct {
     void *k_pages, *v_pages;
     const int32_t* page_table;   // device [n_slots][max_pages]; logical page j of a slot lies at column j % ring_pages
     int32_t n_pages, max_pages, ring_pages, n_kv_heads, head_dim, v_head_dim, window, kv_writes;
+    int32_t keep_first;          // with a window: the first tokens that every query sees beside it (picolm_kv_group)
     const int32_t* write_pages;  // device [n_tokens]: the physical page that takes each new token's key and value
     // with PICOLM_CALL_ATTENDS: the decode step's work list over that group's pages (see
     // picolm_attn_decode_generic in api.h), or the prefill step's tiles of `tile_rows` new tokens
@@ -152,10 +153,11 @@ typedef struct {
 // of a key (0: the same); the ATTENTION operation takes one size for both, a called operation any.
 // keeps_all = 1 with a window: every key stays in its page (no ring) and the window only bounds
 // what a query's work list and tiles visit; a called operation on such a group sees steps of any
-// length.
+// length.  keep_first > 0, with keeps_all and a window: a decode step's work list covers the pages of
+// the sequence's first keep_first tokens too, ahead of the window's.
 typedef struct {
     int32_t n_entries, n_kv_heads, head_dim, window, v_head_dim;
-    int32_t keeps_all;
+    int32_t keeps_all, keep_first;
 } picolm_kv_group;
 
 // Fixed-size state per sequence for `n_entries` layer calls, zeroed when a slot is given out.

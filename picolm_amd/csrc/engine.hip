@@ -106,6 +106,10 @@ struct KVGroup {
     int missing(int slot, int n_tokens) const { return std::max(0, need(n_tokens) - (int)pages[slot].size()); }
     // the first page that a query at `pos` sees
     int first_page(int pos) const { return spec.window > 0 ? std::max(0, pos - spec.window + 1) / PAGE_TOKENS : 0; }
+    // pages ahead of that one which it sees all the same, and how many it sees in all; the n-th of them
+    int kept_pages(int pos) const { return spec.keep_first > 0 ? std::min(pages_for(spec.keep_first), first_page(pos)) : 0; }
+    int seen_pages(int pos) const { return pos / PAGE_TOKENS + 1 - first_page(pos) + kept_pages(pos); }
+    int seen_page(int pos, int n) const { return n < kept_pages(pos) ? n : first_page(pos) + n - kept_pages(pos); }
 };
 
 struct StateGroup {
@@ -261,12 +265,12 @@ static int decode_pages_per_chunk(const std::vector<int>& pos0, int blocks_per_c
 }
 
 // The work list of a decode step over one group's pages: every sequence's visible pages (those of
-// its last `window` keys, or all) cut into runs of `ppc`; an entry is {sequence, which chunk,
+// its last `window` keys and its kept first tokens, or all) cut into runs of `ppc`; an entry is {sequence, which chunk,
 // position of the new token, slot, physical pages of the chunk's first four pages or -1}.  The
 // chunks with the most pages come first: workgroups are handed out in the list's order, and the
 // short last chunks then fill the gaps at the end.
 // Returns the number of entries written behind the header at `out`; *most: chunks of the longest.
-static int chunks_of(const KVGroup& g, int pos, int ppc) { return (pos / PAGE_TOKENS + 1 - g.first_page(pos) + ppc - 1) / ppc; }
+static int chunks_of(const KVGroup& g, int pos, int ppc) { return (g.seen_pages(pos) + ppc - 1) / ppc; }
 
 static int fill_chunk_list(int32_t* out, const std::vector<int>& slots, const std::vector<int>& pos0, int ppc,
                            const KVGroup& g, int* most) {
@@ -276,10 +280,9 @@ static int fill_chunk_list(int32_t* out, const std::vector<int>& slots, const st
     std::vector<Chunk> chunks;
     int longest = 0;
     for (int i = 0; i < (int)slots.size(); ++i) {
-        const int first = g.first_page(pos0[i]), end = pos0[i] / PAGE_TOKENS + 1;
-        const int n = (end - first + ppc - 1) / ppc;
+        const int seen = g.seen_pages(pos0[i]), n = (seen + ppc - 1) / ppc;
         longest = std::max(longest, n);
-        for (int c = 0; c < n; ++c) chunks.push_back({i, c, std::min(end - first - c * ppc, ppc)});
+        for (int c = 0; c < n; ++c) chunks.push_back({i, c, std::min(seen - c * ppc, ppc)});
     }
     std::stable_sort(chunks.begin(), chunks.end(), [](const Chunk& a, const Chunk& b) { return a.n_pages > b.n_pages; });
     out[0] = (int)chunks.size();
@@ -287,15 +290,15 @@ static int fill_chunk_list(int32_t* out, const std::vector<int>& slots, const st
     for (size_t x = 0; x < chunks.size(); ++x) {
         const Chunk& c = chunks[x];
         int32_t* e = out + 8 * (x + 1);
-        const int slot = slots[c.seq], first = g.first_page(pos0[c.seq]), end = pos0[c.seq] / PAGE_TOKENS + 1;
+        const int slot = slots[c.seq], pos = pos0[c.seq], seen = g.seen_pages(pos);
         e[0] = c.seq;
         e[1] = c.idx;
         e[2] = pos0[c.seq];
         e[3] = slot;
         for (int w = 0; w < 4; ++w) {
-            const int page = first + c.idx * ppc + w;
-            const bool inside = page < end && w < ppc;
-            e[4 + w] = inside ? g.table_host[(size_t)slot * g.max_pages + page % g.ring_pages] : -1;
+            const int nth = c.idx * ppc + w;
+            const bool inside = nth < seen && w < ppc;
+            e[4 + w] = inside ? g.table_host[(size_t)slot * g.max_pages + g.seen_page(pos, nth) % g.ring_pages] : -1;
         }
     }
     *most = longest;
@@ -566,6 +569,8 @@ extern "C" int picolm_engine_create(const picolm_program* program, int64_t max_t
         g.spec = program->kv_groups[gi];
         E_REQUIRE(-1, g.spec.n_entries > 0 && g.spec.n_kv_heads > 0 && g.spec.head_dim > 0 && g.spec.window >= 0 && g.spec.v_head_dim >= 0,
                   "engine: cache group %d is ill-formed", gi);
+        E_REQUIRE(-1, g.spec.keep_first >= 0 && (!g.spec.keep_first || (g.spec.keeps_all && g.spec.window > 0)),
+                  "engine: cache group %d keeps %d first tokens; that takes a window and a group that keeps every key", gi, g.spec.keep_first);
         g.max_pages = e->max_pages;
         // a window's ring: the window of the first query of a chunk of new tokens together with the
         // whole chunk, which is written before its queries are answered
@@ -1242,6 +1247,7 @@ static int run_call(Run& r, const picolm_op& o) {
         v.v_head_dim = g.value_dim();
         v.window = g.spec.window;
         v.kv_writes = o.kv_writes;
+        v.keep_first = g.spec.keep_first;
         if (o.kv_writes) v.write_pages = p.at(p.write_pages[o.kv_group]);
         if (o.call_flags & PICOLM_CALL_ATTENDS) {
             if (p.is_decode) {

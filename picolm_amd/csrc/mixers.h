@@ -28,7 +28,8 @@ int picolm_call_loop_input(void* user, const picolm_step_view* v);
 // Softmax attention over the cache entry with biases of the projections, a rotation by position, a
 // norm of queries and keys, a bias by distance, a sink and an output gate, each optional.  A token's
 // q and k are prepared in this order: the projection's bias is added, the first rot_dims entries are
-// turned by the position, the norm is taken; values only get their bias.
+// turned by the position, the norm is taken; values only get their bias.  With norm_all the norm covers
+// all heads of q (and all heads of k) at once and is taken before the rotation.
 //   in: float rows [in_stride] holding q [H d], k [G d], v [G dv] and the gate's pre-activations
 //   [H dv] at the offsets named (v_off may name the keys' place: the values are then the keys as
 //   projected); out: rows [H dv] in the engine's dtype (float with out_float); extra[0]: scratch rows
@@ -63,6 +64,13 @@ typedef struct {
     const float* cos_table;  // [table_positions][rot_dims / 2]; null: no rotation
     const float* sin_table;
     int32_t table_positions, rot_dims, rot_half;      // rot_half = 1: entry i pairs with i + rot_dims / 2; 0: entry 2i with 2i + 1
+    int32_t norm_all;        // 1: q_norm [H head_dim] and k_norm [G head_dim] weigh one norm over all heads, ahead of the rotation (one map)
+    int32_t keep_first;      // a query sees the sequence's first keep_first keys beside its window (as many as the cache entry keeps)
+    float softcap;           // > 0: a scaled score s becomes softcap tanh(s / softcap) (no bias by distance then)
+    int32_t gate_per_head;   // 1: the gate's pre-activations are one a head, [H] at gate_off
+    int32_t first_col;       // the input row's column that q_off, k_off, v_off, gate_off, in_bias and in_stride's end count from
+    int32_t out_stride, out_off;     // out_stride > 0: elements from one output row to the next (0: H maps dv); the heads' outputs,
+    float out_mult;                  // times out_mult, lie at out_off of it
 } picolm_sink_attention_args;
 int picolm_call_sink_attention(void* user, const picolm_step_view* v);
 
@@ -106,16 +114,19 @@ typedef struct {
 int picolm_call_state_scan(void* user, const picolm_step_view* v);
 #define PICOLM_STATE_SCAN_MAX_KEY_DIM 256
 
-// RMS norm in equal parts of a row with a gate of silu(g):
-//   gate_first = 0:  y = x / rms(x) * weight * silu(g);   gate_first = 1:  y = (x silu(g)) / rms(x silu(g)) * weight
-//   the mean is over each part of `group` columns; weight[c % weight_len].
+// RMS norm in equal parts of a row with a gate of act(g), act = silu, or sigmoid with gate_act = 2:
+//   gate_first = 0:  y = x / rms(x) * weight * act(g);   gate_first = 1:  y = (x act(g)) / rms(x act(g)) * weight
+//   the mean is over each part of `group` columns; weight[c % weight_len] (null: one).
 //   in: float rows [width]; extra[0]: float rows [gate_stride], g at gate_off; out: rows [width] in
-//   the engine's dtype.
+//   the engine's dtype; with out_stride > 0 `width` columns at out_off of rows [out_stride], times mult.
 typedef struct {
     const float* weight;
     int32_t weight_len, width, group;
     float eps;
     int32_t gate_first, gate_stride, gate_off;
+    int32_t gate_act;        // 0 or 1: silu, 2: sigmoid
+    int32_t out_stride, out_off;
+    float mult;
 } picolm_gated_norm_args;
 int picolm_call_gated_norm(void* user, const picolm_step_view* v);
 
@@ -217,6 +228,31 @@ typedef struct {
 } picolm_gated_postnorm_args;
 int picolm_call_gated_postnorm(void* user, const picolm_step_view* v);
 
+// A decay per key channel from a product of low rank:
+//   a[c] = sigmoid(z[c])^power,  z = W low + bias,  all in float
+//   in: float rows [in_stride], low [rank] at in_off; out: float rows [channels].
+typedef struct {
+    const float* weight;     // [rank][channels]: W transposed, so that adjacent channels lie side by side
+    const float* bias;       // [channels] or null
+    int32_t channels, rank, in_stride, in_off;
+    float power;
+} picolm_channel_decays_args;
+int picolm_call_channel_decays(void* user, const picolm_step_view* v);
+
+// A branch joins the residual rows behind a norm of its own, and the norm that meets the rows next
+// is taken in the same pass:
+//   x <- x + n(u + bias) * weight;   h = n(x) * next_weight         n(y) = y / sqrt(mean(y^2) + eps)
+//   in: u float rows [width]; out: x float rows [width]; extra[0] (with next_weight): h, rows [width] in
+//   the engine's dtype.
+typedef struct {
+    const float* bias;       // [width] or null
+    const float* weight;     // [width]
+    const float* next_weight;  // [width] or null
+    int32_t width;
+    float eps, next_eps;
+} picolm_branch_norm_args;
+int picolm_call_branch_norm(void* user, const picolm_step_view* v);
+
 // What a matrix state with a forget gate per key channel needs of a token, from pre-activations:
 //   q = silu(q_raw);  a = lower + (1 - lower) sigmoid(f_raw + bias);  k = 1 - a
 //   in: float rows [in_stride], q_raw and f_raw [channels] at q_off, f_off; out: float rows
@@ -233,8 +269,11 @@ int picolm_call_forget_gates(void* user, const picolm_step_view* v);
 //   S[i][j] <- a[i][j] S[i][j] + k[i] w[j];   o[j] = sum_i S[i][j] q[i] + skip[j] x[j]
 //   kind 1: a[i][j] = a[i], a row's decay, given per token and key head; w = x
 //   kind 2: a[i][j] = exp(dt[j] A[j][i]), dt = softplus(dt_raw + dt_bias) per value channel; w = dt x
+//   kind 3: a[i][j] = A[head], a fixed decay per head (between nought and one); w = x
+// With act = 1, q, k and x pass a silu as they are read; then q is multiplied by q_scale and k by
+// k_scale (0: one).
 //   extra[0]: float rows [qk_stride] with q, k (and kind 1: a) [key_heads][key_dim] at q_off, k_off,
-//   a_off; in: float rows [x_stride] with x [heads value_dim] at x_off; extra[1] (kind 2): float
+//   a_off (kind 1 with dt_stride > 0: a lies in extra[1], float rows [dt_stride], at dt_off); in: float rows [x_stride] with x [heads value_dim] at x_off; extra[1] (kind 2): float
 //   rows [dt_stride] with dt_raw [heads value_dim] at dt_off; out: float rows [heads value_dim].
 //   Head h uses q/k head h / (heads / key_heads).
 typedef struct {
@@ -244,9 +283,11 @@ typedef struct {
     int32_t x_stride, x_off;
     int32_t dt_stride, dt_off;
     const float* dt_bias;    // [heads value_dim] or null
-    const float* A;          // kind 2: [heads value_dim][key_dim], negative
+    const float* A;          // kind 2: [heads value_dim][key_dim], negative; kind 3: [heads]
     const float* skip;       // [heads value_dim] or null
     int64_t state_off;       // in floats: [heads][key_dim][value_dim]
+    int32_t act;
+    float q_scale, k_scale;
 } picolm_decay_scan_args;
 int picolm_call_decay_scan(void* user, const picolm_step_view* v);
 

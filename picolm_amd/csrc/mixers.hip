@@ -140,6 +140,55 @@ __global__ void qk_norm_store_kernel(QkPrepare a, T* __restrict__ q_out, T* __re
     }
 }
 
+// The same where one norm covers all heads of q (and one all heads of k): a workgroup per token and
+// one of q, k and v.  The norm comes first, then the rotation.
+template <typename T>
+__global__ __launch_bounds__(1024) void qk_norm_all_store_kernel(QkPrepare a, T* __restrict__ q_out, T* __restrict__ k_pages,
+                                                                 T* __restrict__ v_pages) {
+    __shared__ float scratch[16];
+    const size_t row = blockIdx.x;
+    const int G = a.G, d = a.d, dv = a.dv;
+    const float* src = a.in + row * a.in_stride;
+    const int pos = a.tok_pos[row];
+    if (blockIdx.y == 2) {
+        const float* x = src + a.v_off;
+        const float* b = a.in_bias ? a.in_bias + a.v_off : nullptr;
+        T* dst = v_pages + (size_t)a.write_pages[row] * G * dv * PAGE_TOKENS;
+        for (int i = threadIdx.x; i < G * dv; i += blockDim.x)
+            dst[(size_t)(i / dv) * dv * PAGE_TOKENS + v_page_offset(i % dv, pos % PAGE_TOKENS, dv, a.tiled)] = from_f32<T>(b ? x[i] + b[i] : x[i]);
+        return;
+    }
+    const bool is_q = blockIdx.y == 0;
+    const int n = (is_q ? a.H : G) * d, at = is_q ? a.q_off : a.k_off;
+    const float* x = src + at;
+    const float* b = a.in_bias ? a.in_bias + at : nullptr;
+    const float* w = is_q ? a.q_norm : a.k_norm;
+    auto entry = [&](int i) { return b ? x[i] + b[i] : x[i]; };
+    float ssq = 0.f;
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        const float y = entry(i);
+        ssq += y * y;
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + a.eps);
+    const int half = a.rot_dims / 2;
+    const size_t table_row = a.cos_t ? (size_t)min(pos, a.table_positions - 1) * half : 0;
+    T* k_dst = k_pages + (is_q ? 0 : (size_t)a.write_pages[row] * G * PAGE_TOKENS * d);
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        const int head = i / d, c = i - head * d;
+        float y = entry(i) * inv * w[i];
+        if (a.cos_t && c < a.rot_dims) {
+            int j, other;                  // the pair, and its other entry
+            bool first;
+            if (a.rot_half) j = c < half ? c : c - half, first = c < half, other = first ? i + half : i - half;
+            else j = c >> 1, first = (c & 1) == 0, other = first ? i + 1 : i - 1;
+            const float z = entry(other) * inv * w[other], cs = a.cos_t[table_row + j], sn = a.sin_t[table_row + j];
+            y = first ? y * cs - z * sn : y * cs + z * sn;
+        }
+        if (is_q) q_out[row * n + i] = from_f32<T>(y);
+        else k_dst[(size_t)head * PAGE_TOKENS * d + k_page_offset(pos % PAGE_TOKENS, c, d, a.tiled)] = from_f32<T>(y);
+    }
+}
+
 extern "C" int picolm_call_sink_attention(void* user, const picolm_step_view* v) {
     const picolm_sink_attention_args* a = (const picolm_sink_attention_args*)user;
     VIEW_REQUIRE("sink_attention", v);
@@ -151,13 +200,21 @@ extern "C" int picolm_call_sink_attention(void* user, const picolm_step_view* v)
     PICOLM_REQUIRE(G == v->n_kv_heads && d == v->head_dim && dv == v->v_head_dim && v->window >= 0,
                    "sink_attention: the cache entry holds %d heads of %d and %d (window %d), the operation has %d of %d and %d", v->n_kv_heads,
                    v->head_dim, v->v_head_dim, v->window, G, d, dv);
-    PICOLM_REQUIRE(v->in_row_bytes >= a->in_stride * 4 && a->q_off >= 0 && a->q_off + H * d <= a->in_stride && a->k_off >= 0 &&
-                       a->k_off + G * d <= a->in_stride && a->v_off >= 0 && a->v_off + G * dv <= a->in_stride &&
-                       (a->gate_off < 0 || a->gate_off + H * dv <= a->in_stride),
+    const int cols = a->in_stride - a->first_col;
+    PICOLM_REQUIRE(v->in_row_bytes >= a->in_stride * 4 && a->first_col >= 0 && a->q_off >= 0 && a->q_off + H * d <= cols && a->k_off >= 0 &&
+                       a->k_off + G * d <= cols && a->v_off >= 0 && a->v_off + G * dv <= cols &&
+                       (a->gate_off < 0 || a->gate_off + (a->gate_per_head ? H : H * dv) <= cols),
                    "sink_attention: the input rows of %d floats do not hold what the offsets name", a->in_stride);
     PICOLM_REQUIRE(d % maps == 0 && (maps == 1 || (a->gate_off < 0 && !a->bias)),
                    "sink_attention: %d queries a head of %d entries (with several there is no gate and no bias by distance)", maps, d);
-    PICOLM_REQUIRE(v->out_row_bytes >= (int64_t)H * maps * dv * (a->out_float ? 4 : es) && v->extra_row_bytes[0] >= (int64_t)H * maps * d * es,
+    PICOLM_REQUIRE(!a->norm_all || (maps == 1 && a->q_norm && a->k_norm), "sink_attention: a norm over all heads needs both weights and one map a head");
+    PICOLM_REQUIRE(a->keep_first == v->keep_first && a->softcap >= 0.f && !(a->softcap > 0.f && a->bias),
+                   "sink_attention: %d kept first keys over a cache entry that keeps %d, or a cap of %g beside a bias by distance", a->keep_first,
+                   v->keep_first, (double)a->softcap);
+    const int out_stride = a->out_stride ? a->out_stride : H * maps * dv;
+    PICOLM_REQUIRE((a->out_stride > 0 || a->out_off == 0) && a->out_off >= 0 && a->out_off + H * maps * dv <= out_stride, "sink_attention: output rows of %d do not hold %d heads at %d", out_stride,
+                   H * maps, a->out_off);
+    PICOLM_REQUIRE(v->out_row_bytes >= (int64_t)out_stride * (a->out_float ? 4 : es) && v->extra_row_bytes[0] >= (int64_t)H * maps * d * es,
                    "sink_attention: output or scratch rows too short");
     PICOLM_REQUIRE(!v->kv_writes || v->write_pages, "sink_attention: no pages to write to");
     PICOLM_REQUIRE(a->window >= 0 && (v->window <= 0 || a->window <= v->window), "sink_attention: a window of %d keys over a cache entry laid out for %d",
@@ -167,12 +224,20 @@ extern "C" int picolm_call_sink_attention(void* user, const picolm_step_view* v)
                    "sink_attention: a rotation of %d entries of %d, tables for %d positions", a->rot_dims, d / maps, a->table_positions);
     PICOLM_REQUIRE((H + G) * maps + G <= 65535, "sink_attention: %d heads exceed the grid", (H + G) * maps + G);
     if (v->n_tokens <= 0) return 0;
-    const float* in = (const float*)v->in;
+    const float* in = (const float*)v->in + a->first_col;
+    void* out = (char*)v->out + (size_t)a->out_off * (a->out_float ? 4 : es);
     dim3 grid(v->n_tokens, v->kv_writes ? (H + G) * maps + G : H * maps);
     const bool mfma = dt == PICOLM_BF16 && picolm_attn_plain_mfma_takes(d, dv);      // then the pages are in the matrix-core kernel's order
     QkPrepare p = {in, a->in_stride, a->q_off, a->k_off, a->v_off, a->q_norm, a->k_norm, a->eps, a->unit_qk, a->in_bias, a->cos_table,
                    a->sin_table, a->table_positions, a->rot_dims, a->rot_half, v->tok_pos, v->write_pages, H, G, d, dv, maps, mfma};
-    if (dt == PICOLM_F32)
+    if (a->norm_all) {
+        const dim3 whole(v->n_tokens, v->kv_writes ? 3 : 1);
+        const int threads = H * d >= 2048 && v->n_tokens < 256 ? 1024 : 256;
+        if (dt == PICOLM_F32)
+            qk_norm_all_store_kernel<float><<<whole, threads, 0, v->stream>>>(p, (float*)v->extra[0], (float*)v->k_pages, (float*)v->v_pages);
+        else
+            qk_norm_all_store_kernel<bf16_t><<<whole, threads, 0, v->stream>>>(p, (bf16_t*)v->extra[0], (bf16_t*)v->k_pages, (bf16_t*)v->v_pages);
+    } else if (dt == PICOLM_F32)
         qk_norm_store_kernel<float><<<grid, WAVE, 0, v->stream>>>(p, (float*)v->extra[0], (float*)v->k_pages, (float*)v->v_pages);
     else
         qk_norm_store_kernel<bf16_t><<<grid, WAVE, 0, v->stream>>>(p, (bf16_t*)v->extra[0], (bf16_t*)v->k_pages, (bf16_t*)v->v_pages);
@@ -187,25 +252,30 @@ extern "C" int picolm_call_sink_attention(void* user, const picolm_step_view* v)
     x.mask_window = a->window;
     x.mask_chunk = a->chunk;
     x.out_float = a->out_float;
+    x.keep_first = a->keep_first;
+    x.softcap = a->softcap;
+    x.gate_per_head = a->gate_per_head;
+    x.out_stride = a->out_stride;
+    x.out_mult = a->out_mult;
     const int HM = H * maps;
     if (mfma && v->is_decode)
-        return picolm_attn_decode_plain_mfma(v->extra[0], v->k_pages, v->v_pages, v->out, v->partial, v->n_seq, v->chunk_list, v->n_chunks,
+        return picolm_attn_decode_plain_mfma(v->extra[0], v->k_pages, v->v_pages, out, v->partial, v->n_seq, v->chunk_list, v->n_chunks,
                                              v->pages_per_chunk, v->most_chunks, v->seq_pos0, v->page_table, v->max_pages, v->ring_pages, HM,
                                              G, d, v->window, a->scale, &x, v->stream);
     if (mfma) {
         PICOLM_REQUIRE(v->tile_seq && v->tile_rows == picolm_attn_plain_mfma_tile_rows(), "sink_attention: the step has no tiles of %d rows",
                        picolm_attn_plain_mfma_tile_rows());
-        return picolm_attn_prefill_plain_mfma(v->extra[0], v->k_pages, v->v_pages, v->out, v->tile_seq, v->tile_q0, v->n_tiles, v->seq_slot,
+        return picolm_attn_prefill_plain_mfma(v->extra[0], v->k_pages, v->v_pages, out, v->tile_seq, v->tile_q0, v->n_tiles, v->seq_slot,
                                               v->seq_pos0, v->seq_nnew, v->cu_seqlens, v->page_table, v->max_pages, v->ring_pages, HM, G, d,
                                               v->window, a->scale, &x, v->stream);
     }
     if (v->is_decode)
-        return picolm_attn_decode_plain(v->extra[0], v->k_pages, v->v_pages, v->out, v->partial, dt, v->n_seq, v->chunk_list, v->n_chunks,
+        return picolm_attn_decode_plain(v->extra[0], v->k_pages, v->v_pages, out, v->partial, dt, v->n_seq, v->chunk_list, v->n_chunks,
                                         v->pages_per_chunk, v->most_chunks, v->seq_pos0, v->page_table, v->max_pages, v->ring_pages, HM, G, d,
                                         v->window, a->scale, &x, v->stream);
     PICOLM_REQUIRE(v->tile_seq && v->tile_rows == picolm_attn_prefill_tile_rows(), "sink_attention: the step has no tiles of %d rows",
                    picolm_attn_prefill_tile_rows());
-    return picolm_attn_prefill_plain(v->extra[0], v->k_pages, v->v_pages, v->out, dt, v->tile_seq, v->tile_q0, v->n_tiles, v->seq_slot,
+    return picolm_attn_prefill_plain(v->extra[0], v->k_pages, v->v_pages, out, dt, v->tile_seq, v->tile_q0, v->n_tiles, v->seq_slot,
                                      v->seq_pos0, v->seq_nnew, v->cu_seqlens, v->page_table, v->max_pages, v->ring_pages, HM, G, d, v->window,
                                      a->scale, &x, v->stream);
 }
@@ -638,7 +708,7 @@ extern "C" int picolm_call_state_scan(void* user, const picolm_step_view* v) {
 template <typename T>
 __global__ void gated_norm_kernel(const float* __restrict__ x, const float* __restrict__ gate, int gate_stride, int gate_off,
                                   T* __restrict__ out, const float* __restrict__ weight, int weight_len, int width, int group, float eps,
-                                  int gate_first, int64_t n_units) {
+                                  int gate_first, int gate_act, int out_stride, float mult, int64_t n_units) {
     const int64_t unit = (int64_t)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
     const int lane = threadIdx.x % WAVE;
     if (unit >= n_units) return;
@@ -647,20 +717,21 @@ __global__ void gated_norm_kernel(const float* __restrict__ x, const float* __re
     const int c0 = (int)(unit % n_groups) * group;
     const float* xr = x + row * width + c0;
     const float* gr = gate ? gate + row * gate_stride + gate_off + c0 : nullptr;
+    const auto act = [&](float z) { return gate_act == 2 ? sigmoid_f(z) : silu_f(z); };
     float ssq = 0.f;
     for (int c = lane; c < group; c += WAVE) {
         float xv = xr[c];
-        if (gr && gate_first) xv *= silu_f(gr[c]);
+        if (gr && gate_first) xv *= act(gr[c]);
         ssq += xv * xv;
     }
     ssq = wave_sum(ssq);
     const float inv = 1.f / sqrtf(ssq / (float)group + eps);
     for (int c = lane; c < group; c += WAVE) {
         float xv = xr[c];
-        if (gr && gate_first) xv *= silu_f(gr[c]);
-        float y = xv * inv * weight[(c0 + c) % weight_len];
-        if (gr && !gate_first) y *= silu_f(gr[c]);
-        out[row * width + c0 + c] = from_f32<T>(y);
+        if (gr && gate_first) xv *= act(gr[c]);
+        float y = xv * inv * (weight ? weight[(c0 + c) % weight_len] : 1.f);
+        if (gr && !gate_first) y *= act(gr[c]);
+        out[row * out_stride + c0 + c] = from_f32<T>(y * mult);
     }
 }
 
@@ -668,65 +739,68 @@ __global__ void gated_norm_kernel(const float* __restrict__ x, const float* __re
 template <typename T>
 __global__ __launch_bounds__(1024) void gated_norm_wide_kernel(const float* __restrict__ x, const float* __restrict__ gate, int gate_stride,
                                                               int gate_off, T* __restrict__ out, const float* __restrict__ weight,
-                                                              int weight_len, int width, int group, float eps, int gate_first) {
+                                                              int weight_len, int width, int group, float eps, int gate_first,
+                                                              int gate_act, int out_stride, float mult) {
     __shared__ float scratch[16];
     const int n_groups = width / group;
     const size_t row = blockIdx.x / n_groups;
     const int c0 = (int)(blockIdx.x % n_groups) * group;
     const float* xr = x + row * width + c0;
     const float* gr = gate ? gate + row * gate_stride + gate_off + c0 : nullptr;
+    const auto act = [&](float z) { return gate_act == 2 ? sigmoid_f(z) : silu_f(z); };
     float ssq = 0.f;
     for (int c = threadIdx.x; c < group; c += blockDim.x) {
         float xv = xr[c];
-        if (gr && gate_first) xv *= silu_f(gr[c]);
+        if (gr && gate_first) xv *= act(gr[c]);
         ssq += xv * xv;
     }
     ssq = block_sum(ssq, scratch);
     const float inv = 1.f / sqrtf(ssq / (float)group + eps);
     for (int c = threadIdx.x; c < group; c += blockDim.x) {
         float xv = xr[c];
-        if (gr && gate_first) xv *= silu_f(gr[c]);
-        float y = xv * inv * weight[(c0 + c) % weight_len];
-        if (gr && !gate_first) y *= silu_f(gr[c]);
-        out[row * width + c0 + c] = from_f32<T>(y);
+        if (gr && gate_first) xv *= act(gr[c]);
+        float y = xv * inv * (weight ? weight[(c0 + c) % weight_len] : 1.f);
+        if (gr && !gate_first) y *= act(gr[c]);
+        out[row * out_stride + c0 + c] = from_f32<T>(y * mult);
+    }
+}
+
+template <typename T>
+static void gated_norm_launch(const picolm_gated_norm_args* a, const picolm_step_view* v, int64_t n_units) {
+    const float *in = (const float*)v->in, *gate = (const float*)v->extra[0];
+    T* out = (T*)v->out + a->out_off;
+    const int out_stride = a->out_stride ? a->out_stride : a->width;
+    const float mult = a->out_stride ? a->mult : 1.f;
+    if (a->group >= 1024) {
+        // few rows (a decode step): more threads a part, so that a thread's loads, each of which it waits for, are few
+        const int threads = n_units < 1024 ? 1024 : 256;
+        gated_norm_wide_kernel<T><<<(unsigned)n_units, threads, 0, v->stream>>>(in, gate, a->gate_stride, a->gate_off, out, a->weight, a->weight_len,
+                                                                               a->width, a->group, a->eps, a->gate_first, a->gate_act, out_stride,
+                                                                               mult);
+    } else {
+        gated_norm_kernel<T><<<(unsigned)ceil_div64(n_units, 4), 4 * WAVE, 0, v->stream>>>(in, gate, a->gate_stride, a->gate_off, out, a->weight,
+                                                                                          a->weight_len, a->width, a->group, a->eps, a->gate_first,
+                                                                                          a->gate_act, out_stride, mult, n_units);
     }
 }
 
 extern "C" int picolm_call_gated_norm(void* user, const picolm_step_view* v) {
     const picolm_gated_norm_args* a = (const picolm_gated_norm_args*)user;
     VIEW_REQUIRE("gated_norm", v);
-    PICOLM_REQUIRE(a && a->weight && v->in && v->out, "gated_norm: weights or buffers are missing");
-    PICOLM_REQUIRE(a->width > 0 && a->group > 0 && a->width % a->group == 0 && a->weight_len > 0, "gated_norm: a width of %d in parts of %d",
+    PICOLM_REQUIRE(a && v->in && v->out && a->gate_act >= 0 && a->gate_act <= 2, "gated_norm: buffers are missing, or an unknown gate");
+    PICOLM_REQUIRE(a->width > 0 && a->group > 0 && a->width % a->group == 0 && (!a->weight || a->weight_len > 0), "gated_norm: a width of %d in parts of %d",
                    a->width, a->group);
-    PICOLM_REQUIRE(v->in_row_bytes >= a->width * 4 && v->out_row_bytes >= a->width * elem_bytes(v->dtype), "gated_norm: rows too short");
+    const int out_stride = a->out_stride ? a->out_stride : a->width;
+    PICOLM_REQUIRE(v->in_row_bytes >= a->width * 4 && (a->out_stride > 0 || a->out_off == 0) && a->out_off >= 0 && a->out_off + a->width <= out_stride &&
+                       v->out_row_bytes >= (int64_t)out_stride * elem_bytes(v->dtype),
+                   "gated_norm: rows too short");
     PICOLM_REQUIRE(!v->extra[0] || (a->gate_off >= 0 && a->gate_off + a->width <= a->gate_stride && v->extra_row_bytes[0] >= a->gate_stride * 4),
                    "gated_norm: the gate's rows of %d floats do not hold %d at %d", a->gate_stride, a->width, a->gate_off);
     if (v->rows <= 0) return 0;
     const int64_t n_units = (int64_t)v->rows * (a->width / a->group);
     PICOLM_REQUIRE(n_units < (1ll << 31), "gated_norm: %lld workgroups exceed the grid", (long long)n_units);
-    if (a->group >= 1024) {
-        // few rows (a decode step): more threads a part, so that a thread's loads, each of which it waits for, are few
-        const int threads = n_units < 1024 ? 1024 : 256;
-        if (v->dtype == PICOLM_F32)
-            gated_norm_wide_kernel<float><<<(unsigned)n_units, threads, 0, v->stream>>>((const float*)v->in, (const float*)v->extra[0], a->gate_stride,
-                                                                                    a->gate_off, (float*)v->out, a->weight, a->weight_len,
-                                                                                    a->width, a->group, a->eps, a->gate_first);
-        else
-            gated_norm_wide_kernel<bf16_t><<<(unsigned)n_units, threads, 0, v->stream>>>((const float*)v->in, (const float*)v->extra[0],
-                                                                                     a->gate_stride, a->gate_off, (bf16_t*)v->out, a->weight,
-                                                                                     a->weight_len, a->width, a->group, a->eps, a->gate_first);
-        PICOLM_LAUNCH_CHECK("gated_norm (wide)");
-        return 0;
-    }
-    const int64_t blocks = ceil_div64(n_units, 4);
-    if (v->dtype == PICOLM_F32)
-        gated_norm_kernel<float><<<(unsigned)blocks, 4 * WAVE, 0, v->stream>>>((const float*)v->in, (const float*)v->extra[0], a->gate_stride,
-                                                                               a->gate_off, (float*)v->out, a->weight, a->weight_len, a->width,
-                                                                               a->group, a->eps, a->gate_first, n_units);
-    else
-        gated_norm_kernel<bf16_t><<<(unsigned)blocks, 4 * WAVE, 0, v->stream>>>((const float*)v->in, (const float*)v->extra[0], a->gate_stride,
-                                                                                a->gate_off, (bf16_t*)v->out, a->weight, a->weight_len,
-                                                                                a->width, a->group, a->eps, a->gate_first, n_units);
+    if (v->dtype == PICOLM_F32) gated_norm_launch<float>(a, v, n_units);
+    else gated_norm_launch<bf16_t>(a, v, n_units);
     PICOLM_LAUNCH_CHECK("gated_norm");
     return 0;
 }

@@ -396,6 +396,125 @@ extern "C" int picolm_call_gated_postnorm(void* user, const picolm_step_view* v)
     return 0;
 }
 
+// ---- a branch meets the residual rows behind its norm, and the next norm is taken ------------------------
+// One workgroup a row; a thread's entries of the branch and of the row stay in its registers between
+// the passes where a row has at most BN_KEEP of them a thread.
+#define BN_KEEP 8
+template <typename T>
+__global__ __launch_bounds__(1024) void branch_norm_kernel(float* __restrict__ x, const float* __restrict__ u, T* __restrict__ h,
+                                                           picolm_branch_norm_args a) {
+    __shared__ float scratch[16];
+    const size_t row = blockIdx.x;
+    const int W = a.width;
+    float* xr = x + row * W;
+    const float* ur = u + row * W;
+    float uk[BN_KEEP], xk[BN_KEEP];
+    auto branch_at = [&](int c) { return a.bias ? ur[c] + a.bias[c] : ur[c]; };
+    float ssq = 0.f;
+#pragma unroll
+    for (int i = 0; i < BN_KEEP; ++i) {
+        const int c = threadIdx.x + i * blockDim.x;
+        uk[i] = c < W ? branch_at(c) : 0.f;
+        xk[i] = c < W ? xr[c] : 0.f;
+        ssq += uk[i] * uk[i];
+    }
+    for (int c = threadIdx.x + BN_KEEP * blockDim.x; c < W; c += blockDim.x) {
+        const float y = branch_at(c);
+        ssq += y * y;
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)W + a.eps);
+    float next = 0.f;
+#pragma unroll
+    for (int i = 0; i < BN_KEEP; ++i) {
+        const int c = threadIdx.x + i * blockDim.x;
+        if (c < W) {
+            xk[i] += uk[i] * inv * a.weight[c];
+            xr[c] = xk[i];
+            next += xk[i] * xk[i];
+        }
+    }
+    for (int c = threadIdx.x + BN_KEEP * blockDim.x; c < W; c += blockDim.x) {
+        const float y = xr[c] + branch_at(c) * inv * a.weight[c];
+        xr[c] = y;                                                 // a thread writes what only it reads
+        next += y * y;
+    }
+    if (!a.next_weight) return;                    // (the same for every thread of the grid)
+    const float next_inv = 1.f / sqrtf(block_sum(next, scratch) / (float)W + a.next_eps);
+#pragma unroll
+    for (int i = 0; i < BN_KEEP; ++i) {
+        const int c = threadIdx.x + i * blockDim.x;
+        if (c < W) h[row * W + c] = from_f32<T>(xk[i] * next_inv * a.next_weight[c]);
+    }
+    for (int c = threadIdx.x + BN_KEEP * blockDim.x; c < W; c += blockDim.x) h[row * W + c] = from_f32<T>(xr[c] * next_inv * a.next_weight[c]);
+}
+
+extern "C" int picolm_call_branch_norm(void* user, const picolm_step_view* v) {
+    const picolm_branch_norm_args* a = (const picolm_branch_norm_args*)user;
+    VIEW_REQUIRE("branch_norm", v);
+    PICOLM_REQUIRE(a && a->weight && a->width > 0 && v->in && v->out && v->in != v->out && (!a->next_weight || v->extra[0]),
+                   "branch_norm: weights or buffers are missing");
+    PICOLM_REQUIRE(v->in_row_bytes >= a->width * 4 && v->out_row_bytes >= a->width * 4 &&
+                       (!a->next_weight || v->extra_row_bytes[0] >= a->width * elem_bytes(v->dtype)),
+                   "branch_norm: rows too short for a width of %d", a->width);
+    if (v->rows <= 0) return 0;
+    const int threads = a->width > BN_KEEP * 256 || (v->rows < 256 && a->width >= 1024) ? 1024 : 256;
+    if (v->dtype == PICOLM_F32)
+        branch_norm_kernel<float><<<v->rows, threads, 0, v->stream>>>((float*)v->out, (const float*)v->in, (float*)v->extra[0], *a);
+    else
+        branch_norm_kernel<bf16_t><<<v->rows, threads, 0, v->stream>>>((float*)v->out, (const float*)v->in, (bf16_t*)v->extra[0], *a);
+    PICOLM_LAUNCH_CHECK("branch_norm");
+    return 0;
+}
+
+// ---- a decay per key channel from a product of low rank ------------------------------------------------
+// A workgroup takes CD_ROWS rows by 256 channels: the rows' low parts wait in LDS, a thread keeps a
+// channel's weights for all of them.  sigmoid(z)^power = exp(-power log(1 + e^-z)).
+#define CD_ROWS 8
+__global__ __launch_bounds__(256) void channel_decays_kernel(const float* __restrict__ in, float* __restrict__ out, picolm_channel_decays_args a,
+                                                             int n_rows) {
+    extern __shared__ float cd_low[];      // [rank][CD_ROWS]
+    const int row0 = blockIdx.x * CD_ROWS, c = blockIdx.y * blockDim.x + threadIdx.x;
+    for (int idx = threadIdx.x; idx < CD_ROWS * a.rank; idx += blockDim.x) {
+        const int r = idx % CD_ROWS, i = idx / CD_ROWS;
+        cd_low[idx] = row0 + r < n_rows ? in[(size_t)(row0 + r) * a.in_stride + a.in_off + i] : 0.f;
+    }
+    __syncthreads();
+    if (c >= a.channels) return;
+    float z[CD_ROWS];
+    const float bias = a.bias ? a.bias[c] : 0.f;
+#pragma unroll
+    for (int r = 0; r < CD_ROWS; ++r) z[r] = bias;
+#pragma unroll 4
+    for (int i = 0; i < a.rank; ++i) {
+        const float w = a.weight[(size_t)i * a.channels + c];
+#pragma unroll
+        for (int r = 0; r < CD_ROWS; ++r) z[r] = fmaf(w, cd_low[i * CD_ROWS + r], z[r]);
+    }
+#pragma unroll
+    for (int r = 0; r < CD_ROWS; ++r)
+        if (row0 + r < n_rows) {
+            const float y = -z[r], sp = y > 20.f ? y : log1pf(expf(y));
+            out[(size_t)(row0 + r) * a.channels + c] = expf(-a.power * sp);
+        }
+}
+
+extern "C" int picolm_call_channel_decays(void* user, const picolm_step_view* v) {
+    const picolm_channel_decays_args* a = (const picolm_channel_decays_args*)user;
+    VIEW_REQUIRE("channel_decays", v);
+    PICOLM_REQUIRE(a && a->weight && v->in && v->out && v->in != v->out && a->channels > 0 && a->rank > 0 && a->power > 0.f,
+                   "channel_decays: weights or buffers are missing");
+    PICOLM_REQUIRE(a->in_off >= 0 && a->in_off + a->rank <= a->in_stride && v->in_row_bytes >= a->in_stride * 4 &&
+                       v->out_row_bytes >= a->channels * 4,
+                   "channel_decays: rows too short for a rank of %d and %d channels", a->rank, a->channels);
+    const size_t lds = sizeof(float) * CD_ROWS * (size_t)a->rank;
+    PICOLM_REQUIRE(lds <= 64 * 1024 && ceil_div(a->channels, 256) <= 65535, "channel_decays: a rank of %d needs %zu bytes of LDS", a->rank, lds);
+    if (v->rows <= 0) return 0;
+    channel_decays_kernel<<<dim3(ceil_div(v->rows, CD_ROWS), ceil_div(a->channels, 256)), 256, lds, v->stream>>>((const float*)v->in, (float*)v->out,
+                                                                                                               *a, v->rows);
+    PICOLM_LAUNCH_CHECK("channel_decays");
+    return 0;
+}
+
 // ---- what a forget gate per key channel gives a token --------------------------------------------------
 __global__ void forget_gates_kernel(const float* __restrict__ in, int in_stride, int q_off, int f_off, float* __restrict__ out,
                                     const float* __restrict__ lower, const float* __restrict__ bias, int C, int64_t n) {

@@ -45,6 +45,7 @@ class StepView(Structure):
         ("k_pages", c_void_p), ("v_pages", c_void_p), ("page_table", c_void_p),
         ("n_pages", c_int32), ("max_pages", c_int32), ("ring_pages", c_int32), ("n_kv_heads", c_int32),
         ("head_dim", c_int32), ("v_head_dim", c_int32), ("window", c_int32), ("kv_writes", c_int32),
+        ("keep_first", c_int32),
         ("write_pages", c_void_p),
         ("chunk_list", c_void_p), ("n_chunks", c_int32), ("pages_per_chunk", c_int32), ("most_chunks", c_int32),
         ("partial", c_void_p), ("counters", c_void_p),
@@ -76,7 +77,7 @@ class Op(Structure):
 
 class KVGroup(Structure):
     _fields_ = [("n_entries", c_int32), ("n_kv_heads", c_int32), ("head_dim", c_int32), ("window", c_int32),
-                ("v_head_dim", c_int32), ("keeps_all", c_int32)]
+                ("v_head_dim", c_int32), ("keeps_all", c_int32), ("keep_first", c_int32)]
 
 
 class StateGroup(Structure):
@@ -131,6 +132,7 @@ class ProgramBuilder:
         self.binding = None                   # the cache binding of the layer call being emitted
         self.logits_buffer = -1
         self.failures: list = []              # exceptions that called Python operations raised, newest last
+        self._written_norm = None             # (operations so far, x, weight, eps, buffer): see `note_norm`
         self.labels: dict[int, str] = {}      # operation index -> what a part called it (for timings by operation)
 
     def buffer(self, name: str, width: int, dtype: torch.dtype, rows: int = ROWS_STEP) -> int:
@@ -165,6 +167,16 @@ class ProgramBuilder:
     def rmsnorm(self, norm: NormRef, x: int, out: int, rows: int = ROWS_STEP) -> None:
         self.ops.append(Op(kind=OP_RMSNORM, rows=rows, inp=x, out=out, weight=self._ptr(norm.weight), k=norm.weight.shape[0],
                            eps=norm.eps))
+
+    def note_norm(self, x: int, norm: NormRef, buffer: int) -> None:
+        """The operation just appended has also left the RMSNorm `norm` of the rows in buffer `x` in
+        `buffer`: a part that asks for that norm next, with nothing in between, takes it from there."""
+        self._written_norm = (len(self.ops), x, norm.weight.data_ptr(), norm.eps, buffer)
+
+    def written_norm(self, x: int, norm: NormRef) -> int | None:
+        if self._written_norm is not None and self._written_norm[:4] == (len(self.ops), x, norm.weight.data_ptr(), norm.eps):
+            return self._written_norm[4]
+        return None
 
     def materialize(self, src: Rows, rows: int = ROWS_STEP) -> int:
         """The buffer that holds `src`'s rows, after running the norm they are the result of, if any,
@@ -277,7 +289,7 @@ class BuiltProgram:
         self.failures = b.failures
         self.ops = (Op * len(b.ops))(*b.ops)
         self.buffers = (Buffer * len(b._specs))(*[Buffer(*s) for s in b._specs])
-        kv = [KVGroup(g.n_entries, g.n_kv_heads, g.head_dim, g.window, g.v_head_dim, int(g.keeps_all)) for g in cache_spec.kv_groups]
+        kv = [KVGroup(g.n_entries, g.n_kv_heads, g.head_dim, g.window, g.v_head_dim, int(g.keeps_all), g.keep_first) for g in cache_spec.kv_groups]
         st = [StateGroup(g.n_entries, g.bytes_per_slot) for g in cache_spec.state_groups]
         self.kv_groups = (KVGroup * max(len(kv), 1))(*kv)
         self.state_groups = (StateGroup * max(len(st), 1))(*st)

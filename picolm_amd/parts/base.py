@@ -76,12 +76,14 @@ class Workspace:
 class KVRequest:
     """A mixer's need for keys and values of each token.  `head_dim` is the size of a key;
     `v_head_dim` that of a value where it differs (0: the same).  `keeps_all` with a window: the
-    cache keeps every key (no ring of pages) and the window only bounds what a query visits."""
+    cache keeps every key (no ring of pages) and the window only bounds what a query visits;
+    `keep_first` of the sequence's first tokens are visited too."""
     n_kv_heads: int
     head_dim: int
     window: int = 0
     v_head_dim: int = 0
     keeps_all: bool = False
+    keep_first: int = 0
 
     def __post_init__(self):
         if self.v_head_dim == self.head_dim:        # one way to say "the same": requests compare equal
@@ -313,6 +315,12 @@ class Mixer(Part):
     def emit(self, b, src, x: int, out_norm=None, out_norm_when: int = 0) -> None:
         """x += mixer(src) as operations of a launch program.  This one hands the step to `forward`."""
         _emit_forward(self, b, src, x, *self.cache_requests())
+
+    def emit_branch(self, b, src, out: int):
+        """out = mixer(src) without what it returns: a float row [width] that whoever takes the output
+        adds to every row (a bias of the output projection), or None."""
+        self.emit(b, src, out, accumulate=False)
+        return None
 
 
 class FeedForward(Part):

@@ -217,6 +217,49 @@ class PostNormBlock(Block):
 
 
 
+class SandwichBlock(Block):
+    """A norm ahead of each sublayer and one behind it:
+        x <- x + norm1b(mixer(norm1(x)));   x <- x + norm2b(ffn(norm2(x)))
+    A block without a feed-forward has the first half only.  The norm behind a sublayer, the sum and
+    the norm that meets the rows next (the second half's, or the next block's) are one operation."""
+    graph_safe = True      # launches depend on device memory only
+
+    def __init__(self, mixer_norm: Norm, mixer: Mixer, mixer_after: Norm, ffn_norm: Norm | None, ffn: FeedForward | None,
+                 ffn_after: Norm | None):
+        if (ffn is None) != (ffn_norm is None) or (ffn is None) != (ffn_after is None):
+            raise ValueError("a feed-forward and its two norms come together")
+        self.mixer_norm, self.mixer, self.mixer_after = mixer_norm, mixer, mixer_after
+        self.ffn_norm, self.ffn, self.ffn_after = ffn_norm, ffn, ffn_after
+
+    def children(self):
+        return [p for p in (self.mixer_norm, self.mixer, self.mixer_after, self.ffn_norm, self.ffn, self.ffn_after) if p is not None]
+
+    def first_norm(self):
+        return self.mixer_norm
+
+    def _join(self, b, x: int, branch: int, bias, norm, following) -> None:
+        """x <- x + norm(branch + bias), and the norm `following` of the new x where it is given."""
+        from .calls import BranchNormArgs, emit_library_call
+        ref = norm_ref_of(norm)
+        if ref is None:
+            raise ValueError("a block with norms behind its sublayers takes RMS norms there")
+        extra = [b.buffer("norm.out", norm.size, b.dtype)] if following is not None else []
+        emit_library_call(b, "branch_norm", BranchNormArgs(b._ptr(bias), b._ptr(ref.weight), b._ptr(following.weight if following else None),
+                                                           norm.size, ref.eps, following.eps if following else 0.0), x, inp=branch, extra=extra)
+        if following is not None:
+            b.note_norm(x, following, extra[0])
+
+    def emit(self, b, x: int, after=None, after_when: int = 0) -> None:
+        import torch
+        following = after if after_when == 0 else None
+        branch = b.buffer("sandwich.branch", self.mixer_after.size, torch.float32)
+        bias = self.mixer.emit_branch(b, self.mixer_norm.emit(b, x), branch)
+        self._join(b, x, branch, bias, self.mixer_after, norm_ref_of(self.ffn_norm) if self.ffn is not None else following)
+        if self.ffn is not None:
+            self.ffn.emit(b, self.ffn_norm.emit(b, x), branch, accumulate=False)
+            self._join(b, x, branch, None, self.ffn_after, following)
+
+
 class LoopSum(Block):
     """What runs before pass `number` over a looped stretch of layers where the pass is entered by
     sums alone:  x <- x + x0 (every pass but the first) + step[number], with x0 the embedding's

@@ -18,7 +18,9 @@ class SinkAttentionArgs(Structure):
                 ("scale", c_float), ("eps", c_float),
                 ("q_norm", c_void_p), ("k_norm", c_void_p), ("bias", c_void_p), ("bias_rows", c_int32), ("sink", c_void_p), ("window", c_int32),
                 ("chunk", c_int32), ("maps", c_int32), ("out_float", c_int32), ("unit_qk", c_int32), ("in_bias", c_void_p),
-                ("cos_table", c_void_p), ("sin_table", c_void_p), ("table_positions", c_int32), ("rot_dims", c_int32), ("rot_half", c_int32)]
+                ("cos_table", c_void_p), ("sin_table", c_void_p), ("table_positions", c_int32), ("rot_dims", c_int32), ("rot_half", c_int32),
+                ("norm_all", c_int32), ("keep_first", c_int32), ("softcap", c_float), ("gate_per_head", c_int32), ("first_col", c_int32),
+                ("out_stride", c_int32), ("out_off", c_int32), ("out_mult", c_float)]
 
 
 class ShortConvArgs(Structure):
@@ -37,7 +39,8 @@ class StateScanArgs(Structure):
 
 class GatedNormArgs(Structure):
     _fields_ = [("weight", c_void_p), ("weight_len", c_int32), ("width", c_int32), ("group", c_int32), ("eps", c_float),
-                ("gate_first", c_int32), ("gate_stride", c_int32), ("gate_off", c_int32)]
+                ("gate_first", c_int32), ("gate_stride", c_int32), ("gate_off", c_int32), ("gate_act", c_int32), ("out_stride", c_int32), ("out_off", c_int32),
+                ("mult", c_float)]
 
 
 class NormedSumArgs(Structure):
@@ -87,7 +90,16 @@ class DecayScanArgs(Structure):
     _fields_ = [("kind", c_int32), ("n_heads", c_int32), ("n_key_heads", c_int32), ("key_dim", c_int32), ("value_dim", c_int32),
                 ("qk_stride", c_int32), ("q_off", c_int32), ("k_off", c_int32), ("a_off", c_int32),
                 ("x_stride", c_int32), ("x_off", c_int32), ("dt_stride", c_int32), ("dt_off", c_int32),
-                ("dt_bias", c_void_p), ("A", c_void_p), ("skip", c_void_p), ("state_off", c_int64)]
+                ("dt_bias", c_void_p), ("A", c_void_p), ("skip", c_void_p), ("state_off", c_int64), ("act", c_int32), ("q_scale", c_float), ("k_scale", c_float)]
+
+
+class ChannelDecaysArgs(Structure):
+    _fields_ = [("weight", c_void_p), ("bias", c_void_p), ("channels", c_int32), ("rank", c_int32), ("in_stride", c_int32), ("in_off", c_int32),
+                ("power", c_float)]
+
+
+class BranchNormArgs(Structure):
+    _fields_ = [("bias", c_void_p), ("weight", c_void_p), ("next_weight", c_void_p), ("width", c_int32), ("eps", c_float), ("next_eps", c_float)]
 
 
 class RouteTopArgs(Structure):
@@ -128,7 +140,7 @@ class MapDifferenceArgs(Structure):
 
 
 GATE_NONE, GATE_SILU, GATE_SIGMOID = 0, 1, 2
-DECAY_PER_ROW, DECAY_EXPONENTIAL = 1, 2
+DECAY_PER_ROW, DECAY_EXPONENTIAL, DECAY_FIXED = 1, 2, 3
 DECAY_SCAN_MAX_KEY_DIM = 256
 MAP_RELU_SQUARED, MAP_SOFTCAP, MAP_SCALE = 1, 2, 3
 SCORE_PICKED_SOFTMAX, SCORE_SOFTMAX_ALL, SCORE_SIGMOID = 0, 1, 2

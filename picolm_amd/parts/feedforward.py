@@ -21,13 +21,18 @@ class SwiGLU(FeedForward):
     def children(self):
         return [self.gate_up, self.down]
 
-    def emit(self, b, src, x: int, out_norm=None, out_norm_when: int = 0) -> None:
-        """x += down(silu(gate h) * (up h)) for the rows h of `src`, as operations of a launch program."""
+    def emit(self, b, src, x: int, out_norm=None, out_norm_when: int = 0, accumulate: bool = True) -> None:
+        """x (+)= down(silu(gate h) * (up h)) for the rows h of `src`, as operations of a launch program."""
         if not keeps_forward(self, SwiGLU):
+            if not accumulate:
+                raise ValueError(f"{type(self).__name__} only adds into the rows it is given")
             return FeedForward.emit(self, b, src, x, out_norm, out_norm_when)
         act = b.buffer("ffn.act", self.F, b.dtype)
         self.gate_up.emit(b, src, act, kernels.EPI_SWIGLU)
-        self.down.emit(b, act, x, kernels.EPI_ACCUMULATE, out_norm=out_norm, out_norm_when=out_norm_when)
+        if accumulate:
+            self.down.emit(b, act, x, kernels.EPI_ACCUMULATE, out_norm=out_norm, out_norm_when=out_norm_when)
+        else:
+            self.down.emit(b, act, x, kernels.EPI_STORE)
 
     def forward(self, ctx: StepContext, h, residual) -> None:
         """The same on tensors, now: for parts that run from Python (a routed feed-forward calls

@@ -15,7 +15,8 @@ from .base import Part, Runtime
 
 
 class Linear(Part):
-    """One or several checkpoint matrices stacked along their output rows.
+    """One or several checkpoint matrices stacked along their output rows (a size of -1: as many rows
+    as the checkpoint's tensor has, known once it is loaded).
 
     `interleave=True` stacks exactly two matrices row by row (row 2j of the first, row
     2j+1 of the second): the layout the gated epilogue reads.
@@ -40,6 +41,7 @@ class Linear(Part):
 
     def load(self, fetch, runtime: Runtime) -> None:
         ws = [fetch.get(n) for n in self.names]
+        self.out_sizes = [w.shape[0] if o == -1 else o for w, o in zip(ws, self.out_sizes)]
         self.set_weights(ws, runtime)
 
     def set_weights(self, ws, runtime: Runtime) -> None:
@@ -62,3 +64,20 @@ class Linear(Part):
     def forward(self, a: torch.Tensor, out: torch.Tensor, epilogue: int = kernels.EPI_STORE) -> None:
         """out (=, +=, = silu-gated) a W^T on tensors, now: for parts that run from Python."""
         kernels.gemm(a, self.weight, out, epilogue)
+
+
+class JoinedLinear(Linear):
+    """Checkpoint matrices of one output width side by side along their inputs:
+    y = W_1 x_1 + W_2 x_2 + ... for rows that hold x_1, x_2, ... one after another."""
+
+    def __init__(self, names, out_size: int, in_sizes):
+        super().__init__(names, [out_size], sum(in_sizes))
+        self.in_sizes = list(in_sizes)
+
+    def tensor_specs(self):
+        return [TensorSpec(n, (self.out_sizes[0], k)) for n, k in zip(self.names, self.in_sizes)]
+
+    def set_weights(self, ws, runtime: Runtime) -> None:
+        if runtime.is_f32 or any(w.dtype == torch.float32 for w in ws):
+            ws = [w.to(torch.float32) for w in ws]
+        self.weight = torch.cat(ws, dim=1).contiguous()

@@ -23,6 +23,12 @@ HGRN2, per head a state S [key_dim][value_dim] whose forget gate also weighs wha
     q = silu(W_q h);  v = W_v h;  f = lower + (1 - lower) sigmoid(W_f h + b)                  per head and key channel
     S <- diag(f) S + (1 - f) v^T;  o = S^T q;  out = W_o (rms(o) w_norm)                      rms per head
 
+LinearAttention, per head a state S [key_dim][value_dim] that decays by a fixed factor per head, or per head
+and key channel by one that the token gives:
+    q, k, v = f(W h), f the identity or silu;  q <- q_scale q,  k <- k_scale k
+    S <- diag(a) S + k v^T;  o = S^T q;  a = decay[head], or sigmoid(W_a2 W_a1 h + b)^(1/tau) per key channel
+    out = W_o (rms(o) w_norm act(W_g h))         rms per head or over all heads, w_norm optional, act silu or sigmoid
+
 A mixer's state may lie behind other floats of the layer call's state entry (`state_base`): a
 block that keeps a row of its own there says where the mixer's begins.
 """
@@ -33,8 +39,8 @@ import torch
 from .. import kernels
 from ..weights import TensorSpec
 from .base import Mixer, Runtime, StateRequest
-from .calls import (DECAY_EXPONENTIAL, DECAY_PER_ROW, DECAY_SCAN_MAX_KEY_DIM, GATE_NONE, GATE_SILU, RULE_DELTA, RULE_OUTER_PRODUCT,
-                    SHORT_CONV_MAX_TAPS, STATE_SCAN_MAX_KEY_DIM, DecayScanArgs, ForgetGatesArgs, GatedNormArgs, GateRowsArgs,
+from .calls import (DECAY_EXPONENTIAL, DECAY_FIXED, DECAY_PER_ROW, DECAY_SCAN_MAX_KEY_DIM, GATE_NONE, GATE_SIGMOID, GATE_SILU, RULE_DELTA,
+                    RULE_OUTER_PRODUCT, SHORT_CONV_MAX_TAPS, STATE_SCAN_MAX_KEY_DIM, ChannelDecaysArgs, DecayScanArgs, ForgetGatesArgs, GatedNormArgs, GateRowsArgs,
                     ShortConvArgs, StateScanArgs, emit_library_call)
 from .linear import Linear
 
@@ -285,3 +291,106 @@ class HGRN2(Mixer):
         emit_library_call(b, "gated_norm", GatedNormArgs(b._ptr(self.norm), self.dv, vv, self.dv, self.eps, 0, 0, 0), normed, inp=y)
         self.o.emit(b, normed, x, kernels.EPI_ACCUMULATE if accumulate else kernels.EPI_STORE,
                     **({"out_norm": out_norm, "out_norm_when": out_norm_when} if accumulate else {}))
+
+
+class LinearAttention(Mixer):
+    graph_safe = True      # launches depend on device memory only
+    GATES = {"silu": GATE_SILU, "sigmoid": GATE_SIGMOID}
+
+    def __init__(self, prefix: str, hidden_size: int, n_heads: int, key_dim: int, value_dim: int, eps: float, decay=None, tau: float | None = None,
+                 rank: int | None = None, silu_qkv: bool = False, q_scale: float = 1.0, k_scale: float = 1.0, norm: str = "head",
+                 norm_weight: bool = True, gate: str = "silu"):
+        """`decay`: a factor per head.  Without it the decays are the token's own, per head and key
+        channel, through the tensors a1, a2 and a2.b and the exponent 1/`tau`; `rank`: rows of a1
+        (None: as many as the checkpoint's tensor has).  `silu_qkv`: q, k and v pass a silu.  `norm`:
+        "head" norms every head's output by itself, "all" the heads together; `norm_weight`: with the
+        tensor `norm`, of the size that is normed.  `gate`: the function of W_g h that multiplies the
+        normed outputs."""
+        if not 1 <= key_dim <= DECAY_SCAN_MAX_KEY_DIM:
+            raise ValueError(f"a state with keys of {key_dim}: the kernel takes 1 to {DECAY_SCAN_MAX_KEY_DIM}")
+        if (decay is None) == (tau is None):
+            raise ValueError("decays are fixed (decay) or the token's own (tau)")
+        if decay is not None and (len(decay) != n_heads or not all(0.0 <= x <= 1.0 for x in decay)):
+            raise ValueError(f"decays {list(decay)}: expected one between 0 and 1 for each of {n_heads} heads")
+        if norm not in ("head", "all"):
+            raise ValueError(f"norm '{norm}': known are head, all")
+        if gate not in self.GATES:
+            raise ValueError(f"gate '{gate}': known are {', '.join(self.GATES)}")
+        self.prefix, self.D = prefix, hidden_size
+        self.H, self.dk, self.dv, self.eps = n_heads, key_dim, value_dim, float(eps)
+        self.fixed, self.tau = None if decay is None else [float(x) for x in decay], None if tau is None else float(tau)
+        self.silu_qkv, self.q_scale, self.k_scale = bool(silu_qkv), float(q_scale), float(k_scale)
+        self.norm_group = value_dim if norm == "head" else n_heads * value_dim
+        self.has_norm_weight, self.gate = bool(norm_weight), gate
+        self.state_base = 0
+        self.gives_products = False        # True: a part around this one runs proj and o
+        qk, vv = n_heads * key_dim, n_heads * value_dim
+        names, sizes = ["q", "k", "v", "g"], [qk, qk, vv, vv]
+        if decay is None:
+            names, sizes = names + ["a1"], sizes + [-1 if rank is None else int(rank)]
+        self.proj = Linear([prefix + n for n in names], sizes, hidden_size)
+        self.o = Linear([prefix + "o"], [hidden_size], vv)
+        self.rank = rank
+        self.decay = self.a2 = self.a2_bias = self.norm = None
+
+    def children(self):
+        return [] if self.gives_products else [self.proj, self.o]
+
+    def tensor_specs(self):
+        p, qk = self.prefix, self.H * self.dk
+        specs = [TensorSpec(p + "norm", (self.norm_group,), init="ones")] if self.has_norm_weight else []
+        if self.fixed is None:
+            specs += [TensorSpec(p + "a2", (qk, -1 if self.rank is None else self.rank)), TensorSpec(p + "a2.b", (qk,))]
+        return specs
+
+    def load(self, fetch, runtime: Runtime) -> None:
+        f32 = lambda name: fetch.get(self.prefix + name).to(torch.float32)
+        if self.has_norm_weight:
+            self.norm = f32("norm").contiguous()
+        if self.fixed is not None:
+            self.decay = torch.tensor(self.fixed, dtype=torch.float32, device=runtime.device)
+        else:
+            a1 = fetch.get(self.prefix + "a1")
+            self.a2, self.a2_bias = f32("a2").t().contiguous(), f32("a2.b").contiguous()      # [rank, channels]
+            if self.a2.shape[0] != a1.shape[0]:
+                raise ValueError(f"{self.prefix}a1 has {a1.shape[0]} rows, {self.prefix}a2 takes {self.a2.shape[0]}")
+            self.rank = self.a2.shape[0]
+
+    def state_floats(self) -> int:
+        return self.H * self.dk * self.dv
+
+    def cache_requests(self):
+        return None, StateRequest((self.state_floats(),), torch.float32)
+
+    def emit(self, b, src, x: int, out_norm=None, out_norm_when: int = 0, accumulate: bool = True) -> None:
+        """x (+)= o(norm(scan) * act(g)) for the rows h of `src`, as operations of a launch program."""
+        rows = b.buffer("linear_attn.in", self.proj.out_size, torch.float32)
+        self.proj.emit(b, src, rows, kernels.EPI_STORE)
+        gated = b.buffer("scan.gated", self.heads_width, b.dtype)
+        self.emit_heads(b, rows, self.proj.out_size, 0, gated)
+        self.o.emit(b, gated, x, kernels.EPI_ACCUMULATE if accumulate else kernels.EPI_STORE,
+                    **({"out_norm": out_norm, "out_norm_when": out_norm_when} if accumulate else {}))
+
+    @property
+    def heads_width(self) -> int:
+        return self.H * self.dv
+
+    def emit_heads(self, b, rows: int, stride: int, first_col: int, out: int, out_stride: int = 0, out_off: int = 0, mult: float = 1.0) -> None:
+        """The work between the two projections: `rows` hold the stacked projection's columns from
+        `first_col` on (rows of `stride` floats); the gated outputs go to the rows `out`, or with
+        out_stride > 0, times `mult`, to columns out_off .. of such rows of out_stride entries."""
+        H, qk, vv, at = self.H, self.H * self.dk, self.H * self.dv, first_col
+        y = b.buffer("scan.out", vv, torch.float32)
+        scan = DecayScanArgs(DECAY_FIXED, H, H, self.dk, self.dv, stride, at, at + qk, 0, stride, at + 2 * qk, 0, 0, None, b._ptr(self.decay), None,
+                             self.state_base, int(self.silu_qkv), self.q_scale, self.k_scale)
+        extra = [rows]
+        if self.fixed is None:
+            decays = b.buffer("scan.decays", qk, torch.float32)
+            emit_library_call(b, "channel_decays", ChannelDecaysArgs(b._ptr(self.a2), b._ptr(self.a2_bias), qk, self.rank, stride,
+                                                                     at + 2 * qk + 2 * vv, 1.0 / self.tau), decays, inp=rows)
+            scan.kind, scan.dt_stride = DECAY_PER_ROW, qk
+            extra.append(decays)
+        emit_library_call(b, "decay_scan", scan, y, inp=rows, extra=extra, uses_state=True)
+        norm = GatedNormArgs(b._ptr(self.norm), self.norm_group, vv, self.norm_group, self.eps, 0, stride, at + 2 * qk + vv, self.GATES[self.gate],
+                             out_stride, out_off, mult)
+        emit_library_call(b, "gated_norm", norm, out, inp=y, extra=[rows])
