@@ -318,7 +318,49 @@ def _kekelix_rooflines(cfg: dict, T: int, n_seq: int, context: int) -> dict:
     return {"prefill": pre, "decode": dec}
 
 
+def _zalalix_pair(width: int, heads: int, kv_heads: int, ff: int, gated_ff: int, vocab: int, pairs: int, window: int):
+    """A Zalalix of `pairs` (parallel, fixed-decay) pairs of layers, the second of a pair lightning and
+    retention in turn, with heads of 128 everywhere (the softmax attention over `window` keys and four
+    first ones, half of every head turned and slowed down by wavelength) and gated feed-forwards of
+    `gated_ff`; and the Begopel of the same width, heads, vocabulary and layers, whose feed-forwards of
+    two matrices with `ff` units hold as many weights."""
+    left = dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, softcap=50.0, mask=dict(size=window, keep_first=4),
+                rot=dict(base=500000.0, dims=64, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192)))
+    right = dict(heads=heads, dim=128, vdim=128, tau=16.0, rank=16)
+    fixed = dict(heads=heads, dim=128, vdim=128, decay=[1.0 - 2.0 ** -(3.0 + 6.0 * i / heads) for i in range(heads)])
+    mlp = dict(kind="dense", ff=gated_ff)
+    layers = []
+    for i in range(pairs):
+        layers += [dict(type="parallel", mixer=dict(left=left, left_scale=0.8, right=right, right_scale=1.1), mlp=mlp),
+                   dict(type=("lightning", "retention")[i % 2], mixer=fixed, mlp=mlp)]
+    zal = dict(architecture="Zalalix", vocab=vocab, width=width, embedding=dict(scale=width ** 0.5), norm=dict(eps=1e-5), layers=layers)
+    beg, _ = _begopel_pair(width, heads, kv_heads, ff, vocab, pairs)
+    return zal, beg
+
+
+def _zalalix_rooflines(cfg: dict, T: int, n_seq: int, context: int) -> dict:
+    """As _begopel_rooflines: the attention over the keys that a window and the first tokens show at the
+    bf16 matrix peak, the matrix states at the 32-bit vector peak (5 flops per state element and token;
+    the operation's time covers its decays, norm and gate too);
+    in a decode step the keys and values that are seen and twice the states at HBM's peak."""
+    mfma, valu, hbm = PEAK_TFLOPS["bf16"] * 1e12, PEAK_TFLOPS["fp32"] * 1e12, HBM_PEAK_GBS * 1e9
+    names = ("sink_attention", "linear_attention")
+    pre, dec = {k: 0.0 for k in names}, {k: 0.0 for k in names}
+    for layer in cfg["layers"]:
+        m = layer["mixer"]
+        if layer["type"] == "parallel":
+            l, m = m["left"], m["right"]
+            most = l["mask"]["size"] + l["mask"]["keep_first"]
+            pre["sink_attention"] += 2.0 * l["heads"] * (l["dim"] + l["vdim"]) * sum(min(i + 1, most) for i in range(T)) / mfma
+            dec["sink_attention"] += n_seq * min(context, most) * l["kv_heads"] * (l["dim"] + l["vdim"]) * 2 / hbm
+        pre["linear_attention"] += 5.0 * T * m["heads"] * m["dim"] * m["vdim"] / valu
+        dec["linear_attention"] += n_seq * 2 * m["heads"] * m["dim"] * m["vdim"] * 4 / hbm
+    return {"prefill": pre, "decode": dec}
+
+
 DESIGN_SIZES = {
+    "zalalix": [("width 1024", (1024, 8, 2, 4096, 2752, 32000, 2, 768)), ("width 2048", (2048, 16, 4, 8192, 5504, 32000, 2, 768)),
+                ("width 4096", (4096, 32, 8, 14336, 9600, 128256, 1, 768))],
     "kekelix": [("width 1024", (1024, 8, 1536, 8, 2, 32000, 4)), ("width 2048", (2048, 16, 1536, 8, 2, 32000, 4)),
                 ("width 4096", (4096, 32, 1536, 16, 2, 128256, 3))],
     "begopel": [("width 1024", (1024, 8, 2, 4096, 32000, 2, 2)), ("width 2048", (2048, 16, 4, 8192, 32000, 2, 0)),
@@ -364,7 +406,7 @@ def _zarinex_rooflines(cfg: dict, T: int, n_seq: int, context: int) -> dict:
 def design_comparison(design: str, T: int, n_seq: int, context: int, steps: int) -> dict:
     """Prefill and decode throughput of `design` at a few sizes that resemble real layers (random
     weights), beside the closest model the library has at equal size (for Begopel the Llama, for
-    Zarinex the Begopel, for Satedra the Zarinex, for Kekelix the Satedra), and the GPU time of one prefill step and one decode step by operation."""
+    Zarinex the Begopel, for Satedra the Zarinex, for Kekelix the Satedra, for Zalalix the Begopel), and the GPU time of one prefill step and one decode step by operation."""
     import torch
 
     from picolm_amd.config import LlamaConfig, resolve
@@ -424,6 +466,14 @@ def design_comparison(design: str, T: int, n_seq: int, context: int, steps: int)
 
     for name, size in DESIGN_SIZES[design]:
         print(f"[bench] {design} {name}", file=sys.stderr, flush=True)
+        if design == "zalalix":
+            zal, beg = _zalalix_pair(*size)
+            a = measure(resolve(zal).parse_config(zal), zal["vocab"])
+            b = measure(resolve(beg).parse_config(beg), beg["vocab"])
+            out["sizes"].append({"size": name, "layer_runs": len(zal["layers"]), design: a, "begopel": b,
+                                 "fraction_of_roofline": fractions_of(_zalalix_rooflines(zal, T, n_seq, context), a),
+                                 "begopel_fraction_of_roofline": fractions_of(_begopel_rooflines(beg, T, n_seq, context), b)})
+            continue
         if design == "kekelix":
             kek, sat = _kekelix_pair(*size)
             a = measure(resolve(kek).parse_config(kek), kek["vocab"])

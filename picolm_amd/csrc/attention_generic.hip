@@ -80,7 +80,7 @@ __global__ __launch_bounds__(AT_THREADS) void attn_tile_kernel(AttnArgs a) {
     int page_lo = first_page - kept, page_hi = hi / PAGE_TOKENS + 1;   // [page_lo, page_hi) as counted_page counts them
     if (a.decode) {
         first_page = work.first_page, kept = work.kept_pages;
-        page_lo = kept > 0 ? work.page_lo : max(work.page_lo, seen_lo);
+        page_lo = a.keep_first > 0 ? work.page_lo : max(work.page_lo, seen_lo);
         page_hi = work.page_hi;
     }
 

@@ -120,7 +120,7 @@ __global__ __launch_bounds__(64 * PLAIN_WAVES) void attn_plain_mfma_kernel(AttnA
     // with a window or stretches, the tile of 32 keys that holds the oldest key any query of this wave sees; kept first
     // tokens: their tiles come ahead of those (tiles are counted as counted_page counts, from first_tile - kept_tiles on)
     const int oldest = first_seen(a, qpos_first), my_oldest = first_seen(a, qpos);
-    const int tile_lo = (kept_tiles == 0 ? max(2 * page_lo, oldest / 32) : a.decode ? 2 * page_lo : first_tile - kept_tiles) + (keys_in_turn ? wave : 0);
+    const int tile_lo = (a.keep_first == 0 ? max(2 * page_lo, oldest / 32) : a.decode ? 2 * page_lo : first_tile - kept_tiles) + (keys_in_turn ? wave : 0);
     // two sets of operands in turn: the loads of the tile after this one are queued before this
     // tile's products and stay there (the scheduler may not move them past the barrier), and the
     // page of the tile after that is looked up meanwhile

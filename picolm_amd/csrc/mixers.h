@@ -358,6 +358,21 @@ typedef struct {
 } picolm_map_difference_args;
 int picolm_call_map_difference(void* user, const picolm_step_view* v);
 
+// Linear attention between its projections: the decays of a token (channel_decays, where `decays` has a
+// weight), the matrix state (decay_scan, kind 1 with the decays that were just made or kind 3), the norm
+// and the gate (gated_norm).  In a prompt the three run one after another; in a decode step one kernel
+// does all of it for a sequence and head (a norm over all heads excepted, which follows it).
+//   in: float rows that hold q, k, v, the gate's pre-activations and the decays' low part at the offsets
+//   the three structures name; out: gated rows as gated_norm leaves them; extra[0]: scratch float rows
+//   [heads value_dim]; extra[1] (with decays): scratch float rows [channels].  scan.qk_stride,
+//   scan.x_stride, norm.gate_stride and decays.in_stride are all the input row's length, scan.dt_off 0.
+typedef struct {
+    picolm_channel_decays_args decays;
+    picolm_decay_scan_args scan;
+    picolm_gated_norm_args norm;
+} picolm_linear_attention_args;
+int picolm_call_linear_attention(void* user, const picolm_step_view* v);
+
 // ---- a routed feed-forward ---------------------------------------------------------------------
 // Each row picks `top` of its `experts` router outputs (ties: the lower index).
 //   scoring 0: the largest logits + bias are picked, weighted by the softmax over the picked

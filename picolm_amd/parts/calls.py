@@ -139,6 +139,10 @@ class MapDifferenceArgs(Structure):
     _fields_ = [("heads", c_int32), ("vdim", c_int32), ("out_dtype", c_int32), ("lam", c_float), ("eps", c_float), ("mult", c_float)]
 
 
+class LinearAttentionArgs(Structure):
+    _fields_ = [("decays", ChannelDecaysArgs), ("scan", DecayScanArgs), ("norm", GatedNormArgs)]
+
+
 GATE_NONE, GATE_SILU, GATE_SIGMOID = 0, 1, 2
 DECAY_PER_ROW, DECAY_EXPONENTIAL, DECAY_FIXED = 1, 2, 3
 DECAY_SCAN_MAX_KEY_DIM = 256

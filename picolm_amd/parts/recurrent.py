@@ -41,7 +41,7 @@ from ..weights import TensorSpec
 from .base import Mixer, Runtime, StateRequest
 from .calls import (DECAY_EXPONENTIAL, DECAY_FIXED, DECAY_PER_ROW, DECAY_SCAN_MAX_KEY_DIM, GATE_NONE, GATE_SIGMOID, GATE_SILU, RULE_DELTA,
                     RULE_OUTER_PRODUCT, SHORT_CONV_MAX_TAPS, STATE_SCAN_MAX_KEY_DIM, ChannelDecaysArgs, DecayScanArgs, ForgetGatesArgs, GatedNormArgs, GateRowsArgs,
-                    ShortConvArgs, StateScanArgs, emit_library_call)
+                    LinearAttentionArgs, ShortConvArgs, StateScanArgs, emit_library_call)
 from .linear import Linear
 
 
@@ -380,17 +380,14 @@ class LinearAttention(Mixer):
         `first_col` on (rows of `stride` floats); the gated outputs go to the rows `out`, or with
         out_stride > 0, times `mult`, to columns out_off .. of such rows of out_stride entries."""
         H, qk, vv, at = self.H, self.H * self.dk, self.H * self.dv, first_col
-        y = b.buffer("scan.out", vv, torch.float32)
-        scan = DecayScanArgs(DECAY_FIXED, H, H, self.dk, self.dv, stride, at, at + qk, 0, stride, at + 2 * qk, 0, 0, None, b._ptr(self.decay), None,
-                             self.state_base, int(self.silu_qkv), self.q_scale, self.k_scale)
-        extra = [rows]
+        extra = [b.buffer("scan.out", vv, torch.float32)]
+        args = LinearAttentionArgs()
+        args.scan = DecayScanArgs(DECAY_FIXED, H, H, self.dk, self.dv, stride, at, at + qk, 0, stride, at + 2 * qk, 0, 0, None, b._ptr(self.decay),
+                                  None, self.state_base, int(self.silu_qkv), self.q_scale, self.k_scale)
         if self.fixed is None:
-            decays = b.buffer("scan.decays", qk, torch.float32)
-            emit_library_call(b, "channel_decays", ChannelDecaysArgs(b._ptr(self.a2), b._ptr(self.a2_bias), qk, self.rank, stride,
-                                                                     at + 2 * qk + 2 * vv, 1.0 / self.tau), decays, inp=rows)
-            scan.kind, scan.dt_stride = DECAY_PER_ROW, qk
-            extra.append(decays)
-        emit_library_call(b, "decay_scan", scan, y, inp=rows, extra=extra, uses_state=True)
-        norm = GatedNormArgs(b._ptr(self.norm), self.norm_group, vv, self.norm_group, self.eps, 0, stride, at + 2 * qk + vv, self.GATES[self.gate],
-                             out_stride, out_off, mult)
-        emit_library_call(b, "gated_norm", norm, out, inp=y, extra=[rows])
+            args.decays = ChannelDecaysArgs(b._ptr(self.a2), b._ptr(self.a2_bias), qk, self.rank, stride, at + 2 * qk + 2 * vv, 1.0 / self.tau)
+            args.scan.kind, args.scan.dt_stride = DECAY_PER_ROW, qk
+            extra.append(b.buffer("scan.decays", qk, torch.float32))
+        args.norm = GatedNormArgs(b._ptr(self.norm), self.norm_group, vv, self.norm_group, self.eps, 0, stride, at + 2 * qk + vv,
+                                  self.GATES[self.gate], out_stride, out_off, mult)
+        emit_library_call(b, "linear_attention", args, out, inp=rows, extra=extra, uses_state=True)

@@ -13,10 +13,11 @@ from picolm_amd.parts.base import CacheBinding
 D, H, G, d, V = 64, 4, 2, 16, 100
 
 
-def host_engine(max_tokens=64 * 10, max_seq_len=64 * 4, n_slots=3, layers=2, windows=(0,), v_head_dim=0, state_shape=None):
+def host_engine(max_tokens=64 * 10, max_seq_len=64 * 4, n_slots=3, layers=2, windows=(0,), v_head_dim=0, state_shape=None,
+                keep_first=0, all_groups=False):
     """`layers` attention layers and a head; layer l keeps keys and values in the group of
     windows[l % len(windows)] (0: all keys).  state_shape: also a called operation per layer with a
-    state entry of that shape."""
+    state entry of that shape.  keep_first: groups with a window (all_groups: every group) keep all keys and show the first ones too."""
     b = P.ProgramBuilder(torch.float32, host_only=True)
     x = b.buffer("residual", D, torch.float32)
     b.embed(torch.zeros(V, D), x)
@@ -42,6 +43,7 @@ def host_engine(max_tokens=64 * 10, max_seq_len=64 * 4, n_slots=3, layers=2, win
     lg = b.buffer("logits", V, torch.float32, P.ROWS_WANTED)
     b.linear(torch.zeros(V, D), P.Rows(hf, norm, x), lg, 0, rows=P.ROWS_WANTED)
     b.logits_buffer = lg
-    spec = CacheSpec([KVGroupSpec(n, G, d, w, v_head_dim) for w, n in zip(windows, counts) if n],
+    spec = CacheSpec([KVGroupSpec(n, G, d, w, v_head_dim, keeps_all=keep_first > 0, keep_first=keep_first if w or all_groups else 0)
+                      for w, n in zip(windows, counts) if n],
                      [StateGroupSpec(layers, tuple(state_shape))] if state_shape else [])
     return NativeEngine(b.finish(V, spec), max_tokens, max_seq_len, n_slots, "cpu", host_only=True)

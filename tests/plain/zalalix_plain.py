@@ -118,7 +118,7 @@ def rotate(x, rot, positions=None):
 
 
 def sees(i, j, mask):
-    return j <= i and (i - j < mask["size"] or j < mask["keep_first"])
+    return (j <= i) & ((i - j < mask["size"]) | (j < mask["keep_first"]))
 
 
 def capped(s, cap):
@@ -132,7 +132,7 @@ def softmax_attention(q, k, v, scale, cap, mask):
     G = k.shape[1]
     out = np.zeros((T, H, v.shape[2]))
     for i in range(T):
-        keys = [j for j in range(i + 1) if sees(i, j, mask)]
+        keys = np.flatnonzero(sees(i, np.arange(T), mask))
         for a in range(H):
             g = a // (H // G)
             s = capped(k[keys, g] @ q[i, a] * scale, cap)
@@ -168,19 +168,20 @@ def dense(h, W, p):
     return (silu(h @ W[p + "gate"].T) * (h @ W[p + "up"].T)) @ W[p + "down"].T
 
 
-def forward(config: dict, W: dict, tokens, return_layers: bool = False):
+def forward(config: dict, W: dict, tokens, return_layers: bool = False, touch=lambda rows: rows):
     """logits [T, vocab] of one sequence from its first token; with return_layers also the rows
-    after every layer."""
+    after every layer.  `touch`: what happens to the rows that each sublayer reads (nothing; a test
+    that asks how far small errors spread disturbs them)."""
     W = {k: np.asarray(v, np.float64) for k, v in W.items()}
     eps = config["norm"]["eps"]
     x = W["embed"][np.asarray(tokens)] * config["embedding"]["scale"]
     after = []
     for i, entry in enumerate(config["layers"]):
         p = f"l{i}."
-        y = MIXERS[entry["type"]](rms_norm(x, W[p + "norm1"], eps), W, p + "mix.", entry["mixer"], eps)
+        y = MIXERS[entry["type"]](touch(rms_norm(x, W[p + "norm1"], eps)), W, p + "mix.", entry["mixer"], eps)
         x = x + rms_norm(y, W[p + "norm1b"], eps)
         if entry.get("mlp"):
-            y = dense(rms_norm(x, W[p + "norm2"], eps), W, p + "mlp.")
+            y = dense(touch(rms_norm(x, W[p + "norm2"], eps)), W, p + "mlp.")
             x = x + rms_norm(y, W[p + "norm2b"], eps)
         after.append(x)
     logits = rms_norm(x, W["final.norm"], eps) @ W["head"].T
