@@ -9,11 +9,13 @@
 // chunk's effect on a state is  S_end = P S_start + N  with P the product of the chunk's decays and
 // N the chunk walked from zero; pass 1 leaves (N, P) of every chunk, a second kernel takes the
 // states from chunk to chunk, pass 2 walks every chunk again from its start state and writes the
-// outputs.  The result equals the unchunked walk up to the order of a few products and sums.
+// outputs.  The result equals the unchunked walk up to the order of a few products and sums.  Decays per
+// row and fixed ones have a faster way for prompts, as products on the matrix cores (decay_chunks.hip).
 #include "mixers.h"
 
 #include "api.h"
 #include "common.h"
+#include "decay_scan.h"
 
 #define VIEW_REQUIRE(who, v)                                                                                      \
     PICOLM_REQUIRE((v) && (v)->struct_bytes == (int32_t)sizeof(picolm_step_view), "%s: the step view is of another version", who)
@@ -34,26 +36,6 @@ __device__ __forceinline__ float exp_of_decay(float x) {
 #define DS_TB 16         // tokens whose q, k, decays and inputs wait in LDS at a time
 #define DS_KPT 16        // rows of the state a thread keeps in registers
 #define DS_MAX_KEY_DIM 256
-
-struct DecayScan {
-    const float* qk;
-    const float* x;
-    const float* dt;
-    float* out;
-    float* state;
-    const float* dt_bias;
-    const float* A;
-    const float* skip;
-    const int32_t* cu_seqlens;
-    const int32_t* seq_slot;
-    int64_t slot_floats;
-    int qk_stride, q_off, k_off, a_off, x_stride, x_off, dt_stride, dt_off;
-    int kind, heads, key_heads, key_dim, value_dim, act;
-    float q_scale, k_scale;
-    int R, kpt, n_waves, n_cb;
-    int mode, chunk_len, chunks_per_seq;      // mode 0: whole sequences; 1: (N, P) of every chunk; 3: outputs from the chunks' start states
-    float* ws;                                // [sequence][chunk][head][N | P | S_start][key_dim][value_dim]
-};
 
 __device__ __forceinline__ float* ds_ws(const DecayScan& a, int seq, int chunk, int head, int part) {
     return a.ws + ((((size_t)seq * a.chunks_per_seq + chunk) * a.heads + head) * 3 + part) * a.key_dim * a.value_dim;
@@ -280,6 +262,10 @@ extern "C" int picolm_call_decay_scan(void* user, const picolm_step_view* v) {
     int most_new = 0;
     if (!v->is_decode && !v->recording && v->n_new)
         for (int i = 0; i < v->n_seq; ++i) most_new = std::max(most_new, v->n_new[i]);
+    if (most_new >= PICOLM_DECAY_CHUNKS_FROM && s.kind != 2 && !s.skip && picolm_decay_chunks_ws_floats(s, v->n_seq, most_new) <= DS_WS_LIMIT_FLOATS) {
+        if (ds_workspace(picolm_decay_chunks_ws_floats(s, v->n_seq, most_new), &s.ws)) return -1;
+        return picolm_decay_chunks(s, v->n_seq, most_new, v->stream);
+    }
     if (most_new < DS_CHUNKED_FROM) return launch(v->n_seq);
     s.chunk_len = DS_CHUNK_TOKENS;
     auto ws_floats = [&]() { return (size_t)v->n_seq * ceil_div(most_new, s.chunk_len) * heads * 3 * kd * vd; };
