@@ -324,14 +324,14 @@ def _zalalix_pair(width: int, heads: int, kv_heads: int, ff: int, gated_ff: int,
     first ones, half of every head turned and slowed down by wavelength) and gated feed-forwards of
     `gated_ff`; and the Begopel of the same width, heads, vocabulary and layers, whose feed-forwards of
     two matrices with `ff` units hold as many weights."""
-    left = dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, softcap=50.0, mask=dict(size=window, keep_first=4),
+    left = dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, softcap=30.0, mask=dict(size=window, keep_first=4),
                 rot=dict(base=500000.0, dims=64, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192)))
     right = dict(heads=heads, dim=128, vdim=128, tau=16.0, rank=16)
     fixed = dict(heads=heads, dim=128, vdim=128, decay=[1.0 - 2.0 ** -(3.0 + 6.0 * i / heads) for i in range(heads)])
     mlp = dict(kind="dense", ff=gated_ff)
     layers = []
     for i in range(pairs):
-        layers += [dict(type="parallel", mixer=dict(left=left, left_scale=0.8, right=right, right_scale=1.1), mlp=mlp),
+        layers += [dict(type="parallel", mixer=dict(left=left, left_scale=0.6, right=right, right_scale=1.2), mlp=mlp),
                    dict(type=("lightning", "retention")[i % 2], mixer=fixed, mlp=mlp)]
     zal = dict(architecture="Zalalix", vocab=vocab, width=width, embedding=dict(scale=width ** 0.5), norm=dict(eps=1e-5), layers=layers)
     beg, _ = _begopel_pair(width, heads, kv_heads, ff, vocab, pairs)

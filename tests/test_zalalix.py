@@ -155,7 +155,7 @@ def test_the_plain_rotation_turns_adjacent_entries():
 def test_the_product_side_frequencies_are_the_plain_ones():
     from picolm_amd.config.zalalix import RotationConfig
     from picolm_amd.parts.position import rotary_inv_freq
-    for rot in (dict(base=4.0, dims=8, scaling=zt.slowed(5.0, 1.0, 2.0, 15.0)), dict(base=20000.0, dims=24, scaling=zt.slowed(3.0, 0.5, 7.0, 300)),
+    for rot in (dict(base=4.0, dims=8, scaling=zt.slowed(5.0, 1.0, 2.0, 15.0)), dict(base=30000.0, dims=28, scaling=zt.slowed(3.0, 0.5, 7.0, 300)),
                 dict(base=77.0, dims=6), dict(base=500.0, dims=32, scaling=zt.slowed(2.0, 1.0, 1.0, 100))):
         c = RotationConfig.from_dict(rot, "")
         assert np.allclose(rotary_inv_freq(c.dims, c.base, c.scaling).numpy(), P.rotary_frequencies(rot), rtol=1e-12)

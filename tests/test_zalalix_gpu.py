@@ -112,7 +112,7 @@ ALONE = {
     "lightning, 1,100 columns normed together": one_layer(zt.lightning(16, 220, [0.5, 0.8, 0.9, 0.99, 1.0]), width=64),
     "retention": one_layer(zt.retention(12, 20, [0.9, 0.995])),
     "retention, decays of nought and one": one_layer(zt.retention(7, 3, [1.0, 0.0, 0.5])),
-    "retention, heads of 64": one_layer(zt.retention(64, 64, [0.96875, 0.9995]), width=64),
+    "retention, heads of 64": one_layer(zt.retention(64, 64, [0.9375, 0.9995]), width=64),
     "retention, keys of 200 and values of 1": one_layer(zt.retention(200, 1, [0.9]), width=64),
     "both branches": one_layer(zt.parallel(zt.windowed(4, 2, 12, 10, 0.3, 20, 3, zt.rotation(6)), zt.gla(3, 8, 14, 4.0, 5), 1.4, -0.6)),
     "both branches, heads of 64": one_layer(zt.parallel(zt.windowed(4, 2, 64, 64, 0.15, 20, 3, zt.rotation(32)), zt.gla(2, 64, 96, 4.0, 8)), width=64),

@@ -68,10 +68,10 @@ CONFIG_A = config(211, 72, [
 # 64 to 128); more kept tokens than a page holds, and a window shorter than what is kept
 CONFIG_B = config(515, 256, [
     layer(lightning(64, 32, [0.7, 0.97, 0.9995, 1.0]), 192),
-    layer(parallel(windowed(8, 2, 64, 96, 0.2, 100, 9, rotation(32, 20000.0, slowed(8.0, 1.0, 4.0, 512)), 30.0), gla(4, 48, 40, 16.0, 16)), 320),
+    layer(parallel(windowed(8, 2, 64, 96, 0.2, 100, 9, rotation(32, 30000.0, slowed(8.0, 1.0, 4.0, 512)), 30.0), gla(3, 44, 40, 12.0, 12)), 320),
     layer(parallel(windowed(4, 4, 96, 64, 0.15, 60, 75, rotation(96, 100000.0), 12.0), gla(2, 64, 128, 2.0, 8), 0.9, 1.0), None),
-    layer(retention(32, 64, [0.96875, 0.999, 0.8]), 128),
-    layer(parallel(windowed(8, 1, 128, 128, 0.1, 129, 1, rotation(64, 20000.0)), gla(1, 100, 60, 8.0, 20), 1.0, 0.5), 64),
+    layer(retention(32, 64, [0.9375, 0.999, 0.8]), 128),
+    layer(parallel(windowed(8, 1, 128, 128, 0.1, 129, 1, rotation(64, 30000.0)), gla(1, 100, 60, 8.0, 20), 1.0, 0.5), 64),
 ], scale=16.0)
 
 # C: no size is a multiple of 8; one head; windows of one and two positions; nothing kept; a rank of one; decays of nought and one
