@@ -1,7 +1,8 @@
 // Linear attention between its projections (mixers.h, picolm_call_linear_attention).  A prompt runs the
-// three operations it consists of; a decode step runs one kernel, in which a workgroup has a sequence's
-// head: it makes the token's decays, carries the state over the token, reads it out along q, and norms
-// and gates the head's output.  All arithmetic is float; the state is read and written once.
+// operations it consists of; a decode step runs one kernel, in which a workgroup has a sequence's
+// head: it turns q and k by the token's position, makes the token's decays, carries the state over the
+// token, reads it out along q, and norms and gates the head's output.  All arithmetic is float; the
+// state is read and written once.
 #include "mixers.h"
 
 #include "api.h"
@@ -22,6 +23,7 @@ struct LinearStep {
     float* y;                // not null: the head's raw output goes here, and norm and gate follow in another kernel
     float* state;
     const int32_t* seq_slot;
+    const int32_t* tok_pos;
     int64_t slot_floats;
     int columns;             // threads side by side along a row of the state, a power of two
     picolm_linear_attention_args a;
@@ -50,9 +52,20 @@ __global__ __launch_bounds__(LS_THREADS) void linear_step_kernel(LinearStep s) {
     };
     load(col, group);
     const auto read = [&](float x) { return sc.act ? silu_f(x) : x; };
+    const int half = s.a.rot_dims / 2;
+    const size_t table_row = s.a.cos_table ? (size_t)min(s.tok_pos[seq], s.a.table_positions - 1) * half : 0;
     for (int i = tid; i < kd; i += LS_THREADS) {
-        qs[i] = read(row[sc.q_off + head * kd + i]) * sc.q_scale;
-        ks[i] = read(row[sc.k_off + head * kd + i]) * sc.k_scale;
+        const float *q = row + sc.q_off + head * kd, *k = row + sc.k_off + head * kd;
+        float qv = read(q[i]), kv = read(k[i]);
+        if (s.a.cos_table && i < s.a.rot_dims) {
+            const bool first = s.a.rot_half ? i < half : (i & 1) == 0;
+            const int j = s.a.rot_half ? (first ? i : i - half) : i >> 1, other = s.a.rot_half ? (first ? i + half : i - half) : i ^ 1;
+            const float c = s.a.cos_table[table_row + j], sn = first ? -s.a.sin_table[table_row + j] : s.a.sin_table[table_row + j];
+            qv = qv * c + q[other] * sn;
+            kv = kv * c + k[other] * sn;
+        }
+        qs[i] = qv * sc.q_scale;
+        ks[i] = kv * sc.k_scale;
         float decay;
         if (sc.kind == 3) {
             decay = sc.A[head];
@@ -132,7 +145,15 @@ extern "C" int picolm_call_linear_attention(void* user, const picolm_step_view* 
     PICOLM_REQUIRE(sc.qk_stride == sc.x_stride && a->norm.gate_stride == sc.x_stride && (!made || a->decays.in_stride == sc.x_stride) &&
                        a->norm.width == sc.n_heads * sc.value_dim && !a->norm.gate_first,
                    "linear_attention: the operations' rows differ");
+    PICOLM_REQUIRE(!a->cos_table || (a->sin_table && a->table_positions > 0 && a->rot_dims > 0 && a->rot_dims % 2 == 0 && a->rot_dims <= sc.key_dim &&
+                                     !sc.act && v->tok_pos && v->rows == v->n_tokens),
+                   "linear_attention: a rotation of %d entries of %d, tables for %d positions (it takes no activation)", a->rot_dims, sc.key_dim,
+                   a->table_positions);
     if (v->n_tokens <= 0) return 0;
+    if (a->cos_table)
+        for (int i = 0; i < v->n_seq; ++i)
+            PICOLM_REQUIRE(v->recording || v->pos0[i] + v->n_new[i] <= a->table_positions,
+                           "linear_attention: sequence %d reaches position %d, the tables hold %d", i, v->pos0[i] + v->n_new[i], a->table_positions);
     picolm_step_view w = *v;
     const auto give = [&](void* in, int in_bytes, void* out, int out_bytes, void* e0, int e0_bytes, void* e1, int e1_bytes) {
         w.in = in, w.in_row_bytes = in_bytes, w.out = out, w.out_row_bytes = out_bytes;
@@ -143,6 +164,19 @@ extern "C" int picolm_call_linear_attention(void* user, const picolm_step_view* 
         return picolm_call_gated_norm(&a->norm, &w);
     };
     if (!v->is_decode) {
+        if (a->cos_table) {       // q and k in place: one pass where their heads lie side by side
+            picolm_rotate_heads_args r = {};
+            const bool joined = sc.k_off == sc.q_off + sc.n_heads * sc.key_dim;
+            r.cos_table = a->cos_table, r.sin_table = a->sin_table, r.table_positions = a->table_positions;
+            r.dims = a->rot_dims, r.half = a->rot_half, r.heads = sc.n_heads * (joined ? 2 : 1), r.width = a->rot_dims;
+            r.in_stride = r.out_stride = sc.qk_stride, r.in_head_stride = r.out_head_stride = sc.key_dim;
+            give(v->in, v->in_row_bytes, v->in, v->in_row_bytes, nullptr, 0, nullptr, 0);
+            r.in_off = r.out_off = sc.q_off;
+            if (const int rc = picolm_call_rotate_heads(&r, &w)) return rc;
+            r.in_off = r.out_off = sc.k_off;
+            if (!joined)
+                if (const int rc = picolm_call_rotate_heads(&r, &w)) return rc;
+        }
         if (made) {
             give(v->in, v->in_row_bytes, v->extra[1], v->extra_row_bytes[1], nullptr, 0, nullptr, 0);
             if (const int rc = picolm_call_channel_decays(&a->decays, &w)) return rc;
@@ -174,7 +208,7 @@ extern "C" int picolm_call_linear_attention(void* user, const picolm_step_view* 
     const bool joint = a->norm.group != vd;
     LinearStep s;
     s.in = (const float*)v->in, s.out = v->out, s.y = joint ? (float*)v->extra[0] : nullptr;
-    s.state = (float*)v->state + sc.state_off, s.seq_slot = v->seq_slot, s.slot_floats = v->state_bytes_per_slot / 4;
+    s.state = (float*)v->state + sc.state_off, s.seq_slot = v->seq_slot, s.tok_pos = v->tok_pos, s.slot_floats = v->state_bytes_per_slot / 4;
     s.a = *a;
     if (s.a.scan.q_scale == 0.f) s.a.scan.q_scale = 1.f;
     if (s.a.scan.k_scale == 0.f) s.a.scan.k_scale = 1.f;

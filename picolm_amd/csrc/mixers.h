@@ -37,7 +37,8 @@ int picolm_call_loop_input(void* user, const picolm_step_view* v);
 //   H (dv + 2), tile_rows = picolm_attn_plain_mfma_tile_rows() where the engine runs in bfloat16 and
 //   picolm_attn_plain_mfma_takes(d, dv) (the matrix-core kernel then runs), else
 //   picolm_attn_prefill_tile_rows().  The operation writes its own pages: as plain arrays, or for the
-//   matrix-core kernel in the order of its operands.
+//   matrix-core kernel in the order of its operands.  A layer call that reads another call's entry
+//   writes none, and its k_off, v_off and k_norm are not looked at.
 // maps > 1: a head's d entries are `maps` queries (and a KV head's `maps` keys) of d / maps entries
 //   side by side, each an attention of its own over the same values: query m of a head meets part m of
 //   the cached key.  The attention then runs over H maps heads: out rows [H maps][dv], scratch rows
@@ -71,6 +72,8 @@ typedef struct {
     int32_t first_col;       // the input row's column that q_off, k_off, v_off, gate_off, in_bias and in_stride's end count from
     int32_t out_stride, out_off;     // out_stride > 0: elements from one output row to the next (0: H maps dv); the heads' outputs,
     float out_mult;                  // times out_mult, lie at out_off of it
+    float temp_coef;         // with temp_every > 0 the prepared query of position p is multiplied by
+    double temp_every;       // 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
 } picolm_sink_attention_args;
 int picolm_call_sink_attention(void* user, const picolm_step_view* v);
 
@@ -241,15 +244,18 @@ int picolm_call_channel_decays(void* user, const picolm_step_view* v);
 
 // A branch joins the residual rows behind a norm of its own, and the norm that meets the rows next
 // is taken in the same pass:
-//   x <- x + n(u + bias) * weight;   h = n(x) * next_weight         n(y) = y / sqrt(mean(y^2) + eps)
+//   x <- x + mult n(u + bias) * weight;   h = n(x) * next_weight    n(y) = y / sqrt(mean(y^2) + eps)
 //   in: u float rows [width]; out: x float rows [width]; extra[0] (with next_weight): h, rows [width] in
-//   the engine's dtype.
+//   the engine's dtype.  plain = 1 (without next_weight): h is the new x itself, for the products that
+//   read the rows without a norm.
 typedef struct {
     const float* bias;       // [width] or null
     const float* weight;     // [width]
     const float* next_weight;  // [width] or null
     int32_t width;
     float eps, next_eps;
+    float mult;              // 0: one
+    int32_t plain;
 } picolm_branch_norm_args;
 int picolm_call_branch_norm(void* user, const picolm_step_view* v);
 
@@ -366,10 +372,16 @@ int picolm_call_map_difference(void* user, const picolm_step_view* v);
 //   the three structures name; out: gated rows as gated_norm leaves them; extra[0]: scratch float rows
 //   [heads value_dim]; extra[1] (with decays): scratch float rows [channels].  scan.qk_stride,
 //   scan.x_stride, norm.gate_stride and decays.in_stride are all the input row's length, scan.dt_off 0.
+// With tables, the first rot_dims entries of every head of q and k are turned by the token's position
+// before all that (as in rotate_heads; without scan.act): by the decode step's kernel as it reads them, in a
+// prompt by a pass over the input rows, which are left turned.
 typedef struct {
     picolm_channel_decays_args decays;
     picolm_decay_scan_args scan;
     picolm_gated_norm_args norm;
+    const float* cos_table;  // [table_positions][rot_dims / 2]; null: no rotation
+    const float* sin_table;
+    int32_t table_positions, rot_dims, rot_half;
 } picolm_linear_attention_args;
 int picolm_call_linear_attention(void* user, const picolm_step_view* v);
 
@@ -380,14 +392,15 @@ int picolm_call_linear_attention(void* user, const picolm_step_view* v);
 //   scoring 1: s = softmax over all the logits; the largest s + bias are picked; the weights are
 //              the picked s over their sum (+ 1e-20), times `scale`.
 //   scoring 2: s = sigmoid(logit); the largest s + bias are picked; the weights are the picked s
-//              themselves, times `scale`.
+//              themselves, times `scale`;
+//   scoring 3: s and the picks as in 1, but the weights are the picked s themselves, times `scale`.
 //   in: float rows [in_stride] (0: experts) whose first `experts` entries are the router logits
 //   without bias; out: rows of 2 top words: the picked outputs (int32) and then their weights (float).
 typedef struct {
     const float* bias;       // [experts] or null
     int32_t experts, top;
     int32_t scoring, in_stride;
-    float scale;             // scoring 1
+    float scale;             // scoring 1 to 3
 } picolm_route_top_args;
 int picolm_call_route_top(void* user, const picolm_step_view* v);
 

@@ -64,7 +64,14 @@ struct QkPrepare {
     const int32_t* write_pages;
     int H, G, d, dv, maps;
     bool tiled;
+    float temp_coef;
+    double temp_every;
 };
+
+// the factor on the queries of position pos
+__device__ __forceinline__ float query_temperature(const QkPrepare& a, int pos) {
+    return a.temp_every > 0.0 ? 1.f + a.temp_coef * logf((float)(floor((pos + 1) / a.temp_every) + 1.0)) : 1.f;
+}
 
 // One wave per (token, part): a part is one of the `maps` queries of a query head, one of the `maps`
 // keys of a KV head, or a value head.  Queries go, biased, turned and normed, to the rows the
@@ -111,6 +118,7 @@ __global__ void qk_norm_store_kernel(QkPrepare a, T* __restrict__ q_out, T* __re
         }
         const int m = part % maps, lo = m * dp;
         if (is_q) {
+            const float temp = query_temperature(a, a.tok_pos[row]);
             T* dst = q_out + (row * H * maps + part) * d;
             for (int i = lane; i < d; i += WAVE) {
                 float y = 0.f;
@@ -118,7 +126,7 @@ __global__ void qk_norm_store_kernel(QkPrepare a, T* __restrict__ q_out, T* __re
                     y = value(i - lo);
                     if (norms) y = w ? y * inv * w[i - lo] : y * inv;
                 }
-                dst[i] = from_f32<T>(y);
+                dst[i] = from_f32<T>(y * temp);
             }
         } else {
             const int head = part / maps;
@@ -173,6 +181,7 @@ __global__ __launch_bounds__(1024) void qk_norm_all_store_kernel(QkPrepare a, T*
     const int half = a.rot_dims / 2;
     const size_t table_row = a.cos_t ? (size_t)min(pos, a.table_positions - 1) * half : 0;
     T* k_dst = k_pages + (is_q ? 0 : (size_t)a.write_pages[row] * G * PAGE_TOKENS * d);
+    const float temp = is_q ? query_temperature(a, pos) : 1.f;
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
         const int head = i / d, c = i - head * d;
         float y = entry(i) * inv * w[i];
@@ -184,7 +193,7 @@ __global__ __launch_bounds__(1024) void qk_norm_all_store_kernel(QkPrepare a, T*
             const float z = entry(other) * inv * w[other], cs = a.cos_t[table_row + j], sn = a.sin_t[table_row + j];
             y = first ? y * cs - z * sn : y * cs + z * sn;
         }
-        if (is_q) q_out[row * n + i] = from_f32<T>(y);
+        if (is_q) q_out[row * n + i] = from_f32<T>(y * temp);
         else k_dst[(size_t)head * PAGE_TOKENS * d + k_page_offset(pos % PAGE_TOKENS, c, d, a.tiled)] = from_f32<T>(y);
     }
 }
@@ -201,13 +210,13 @@ extern "C" int picolm_call_sink_attention(void* user, const picolm_step_view* v)
                    "sink_attention: the cache entry holds %d heads of %d and %d (window %d), the operation has %d of %d and %d", v->n_kv_heads,
                    v->head_dim, v->v_head_dim, v->window, G, d, dv);
     const int cols = a->in_stride - a->first_col;
-    PICOLM_REQUIRE(v->in_row_bytes >= a->in_stride * 4 && a->first_col >= 0 && a->q_off >= 0 && a->q_off + H * d <= cols && a->k_off >= 0 &&
-                       a->k_off + G * d <= cols && a->v_off >= 0 && a->v_off + G * dv <= cols &&
+    PICOLM_REQUIRE(v->in_row_bytes >= a->in_stride * 4 && a->first_col >= 0 && a->q_off >= 0 && a->q_off + H * d <= cols &&
+                       (!v->kv_writes || (a->k_off >= 0 && a->k_off + G * d <= cols && a->v_off >= 0 && a->v_off + G * dv <= cols)) &&
                        (a->gate_off < 0 || a->gate_off + (a->gate_per_head ? H : H * dv) <= cols),
                    "sink_attention: the input rows of %d floats do not hold what the offsets name", a->in_stride);
     PICOLM_REQUIRE(d % maps == 0 && (maps == 1 || (a->gate_off < 0 && !a->bias)),
                    "sink_attention: %d queries a head of %d entries (with several there is no gate and no bias by distance)", maps, d);
-    PICOLM_REQUIRE(!a->norm_all || (maps == 1 && a->q_norm && a->k_norm), "sink_attention: a norm over all heads needs both weights and one map a head");
+    PICOLM_REQUIRE(!a->norm_all || (maps == 1 && a->q_norm && (a->k_norm || !v->kv_writes)), "sink_attention: a norm over all heads needs both weights and one map a head");
     PICOLM_REQUIRE(a->keep_first == v->keep_first && a->softcap >= 0.f && !(a->softcap > 0.f && a->bias),
                    "sink_attention: %d kept first keys over a cache entry that keeps %d, or a cap of %g beside a bias by distance", a->keep_first,
                    v->keep_first, (double)a->softcap);
@@ -220,6 +229,7 @@ extern "C" int picolm_call_sink_attention(void* user, const picolm_step_view* v)
     PICOLM_REQUIRE(a->window >= 0 && (v->window <= 0 || a->window <= v->window), "sink_attention: a window of %d keys over a cache entry laid out for %d",
                    a->window, v->window);
     PICOLM_REQUIRE(a->chunk >= 0, "sink_attention: stretches of %d keys", a->chunk);
+    PICOLM_REQUIRE(a->temp_every >= 0.0, "sink_attention: a temperature that steps every %g positions", a->temp_every);
     PICOLM_REQUIRE(!a->cos_table || (a->sin_table && a->table_positions > 0 && a->rot_dims > 0 && a->rot_dims % 2 == 0 && a->rot_dims <= d / maps),
                    "sink_attention: a rotation of %d entries of %d, tables for %d positions", a->rot_dims, d / maps, a->table_positions);
     PICOLM_REQUIRE((H + G) * maps + G <= 65535, "sink_attention: %d heads exceed the grid", (H + G) * maps + G);
@@ -229,7 +239,8 @@ extern "C" int picolm_call_sink_attention(void* user, const picolm_step_view* v)
     dim3 grid(v->n_tokens, v->kv_writes ? (H + G) * maps + G : H * maps);
     const bool mfma = dt == PICOLM_BF16 && picolm_attn_plain_mfma_takes(d, dv);      // then the pages are in the matrix-core kernel's order
     QkPrepare p = {in, a->in_stride, a->q_off, a->k_off, a->v_off, a->q_norm, a->k_norm, a->eps, a->unit_qk, a->in_bias, a->cos_table,
-                   a->sin_table, a->table_positions, a->rot_dims, a->rot_half, v->tok_pos, v->write_pages, H, G, d, dv, maps, mfma};
+                   a->sin_table, a->table_positions, a->rot_dims, a->rot_half, v->tok_pos, v->write_pages, H, G, d, dv, maps, mfma, a->temp_coef,
+                   a->temp_every};
     if (a->norm_all) {
         const dim3 whole(v->n_tokens, v->kv_writes ? 3 : 1);
         const int threads = H * d >= 2048 && v->n_tokens < 256 ? 1024 : 256;

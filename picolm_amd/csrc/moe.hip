@@ -49,8 +49,8 @@ __global__ void route_top_kernel(const float* __restrict__ logits, int in_stride
         }
         return;
     }
-    if (scoring == 1) {
-        // s = softmax over every output; the picks are the largest s + bias, their weights the picked s over their sum
+    if (scoring == 1 || scoring == 3) {
+        // s = softmax over every output; the picks are the largest s + bias, their weights the picked s over their sum or (3) as they are
         float zmax = -INFINITY, den = 0.f;
         for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, z[e]);
         for (int e = 0; e < E; ++e) den += expf(z[e] - zmax);
@@ -70,7 +70,7 @@ __global__ void route_top_kernel(const float* __restrict__ logits, int in_stride
             sum += best_s;
             last_c = best, last_e = be;
         }
-        for (int k = 0; k < top; ++k) w[k] = w[k] / (sum + 1e-20f) * scale;
+        for (int k = 0; k < top; ++k) w[k] = (scoring == 1 ? w[k] / (sum + 1e-20f) : w[k]) * scale;
         return;
     }
     float last_z = INFINITY, first_z = 0.f, sum = 0.f;
@@ -101,7 +101,7 @@ extern "C" int picolm_call_route_top(void* user, const picolm_step_view* v) {
                    a ? a->top : 0, a ? a->experts : 0);
     const int in_stride = a->in_stride ? a->in_stride : a->experts;
     PICOLM_REQUIRE(in_stride >= a->experts && v->in_row_bytes >= (int64_t)in_stride * 4 && v->out_row_bytes >= 2 * a->top * 4, "route_top: rows too short");
-    PICOLM_REQUIRE(a->scoring >= 0 && a->scoring <= 2, "route_top: scoring %d is not known", a->scoring);
+    PICOLM_REQUIRE(a->scoring >= 0 && a->scoring <= 3, "route_top: scoring %d is not known", a->scoring);
     if (v->rows <= 0) return 0;
     route_top_kernel<<<ceil_div(v->rows, 64), 64, 0, v->stream>>>((const float*)v->in, in_stride, a->bias, (int32_t*)v->out, a->experts, a->top,
                                                                  v->rows, a->scoring, a->scale);

@@ -423,19 +423,22 @@ __global__ __launch_bounds__(1024) void branch_norm_kernel(float* __restrict__ x
         ssq += y * y;
     }
     const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)W + a.eps);
+    const float scaled = inv * a.mult;
     float next = 0.f;
 #pragma unroll
     for (int i = 0; i < BN_KEEP; ++i) {
         const int c = threadIdx.x + i * blockDim.x;
         if (c < W) {
-            xk[i] += uk[i] * inv * a.weight[c];
+            xk[i] += uk[i] * scaled * a.weight[c];
             xr[c] = xk[i];
+            if (a.plain) h[row * W + c] = from_f32<T>(xk[i]);
             next += xk[i] * xk[i];
         }
     }
     for (int c = threadIdx.x + BN_KEEP * blockDim.x; c < W; c += blockDim.x) {
-        const float y = xr[c] + branch_at(c) * inv * a.weight[c];
+        const float y = xr[c] + branch_at(c) * scaled * a.weight[c];
         xr[c] = y;                                                 // a thread writes what only it reads
+        if (a.plain) h[row * W + c] = from_f32<T>(y);
         next += y * y;
     }
     if (!a.next_weight) return;                    // (the same for every thread of the grid)
@@ -451,17 +454,20 @@ __global__ __launch_bounds__(1024) void branch_norm_kernel(float* __restrict__ x
 extern "C" int picolm_call_branch_norm(void* user, const picolm_step_view* v) {
     const picolm_branch_norm_args* a = (const picolm_branch_norm_args*)user;
     VIEW_REQUIRE("branch_norm", v);
-    PICOLM_REQUIRE(a && a->weight && a->width > 0 && v->in && v->out && v->in != v->out && (!a->next_weight || v->extra[0]),
-                   "branch_norm: weights or buffers are missing");
+    PICOLM_REQUIRE(a && a->weight && a->width > 0 && v->in && v->out && v->in != v->out && (!(a->next_weight || a->plain) || v->extra[0]) &&
+                       !(a->next_weight && a->plain),
+                   "branch_norm: weights or buffers are missing, or both the rows and their norm are asked for");
     PICOLM_REQUIRE(v->in_row_bytes >= a->width * 4 && v->out_row_bytes >= a->width * 4 &&
-                       (!a->next_weight || v->extra_row_bytes[0] >= a->width * elem_bytes(v->dtype)),
+                       (!(a->next_weight || a->plain) || v->extra_row_bytes[0] >= a->width * elem_bytes(v->dtype)),
                    "branch_norm: rows too short for a width of %d", a->width);
     if (v->rows <= 0) return 0;
     const int threads = a->width > BN_KEEP * 256 || (v->rows < 256 && a->width >= 1024) ? 1024 : 256;
+    picolm_branch_norm_args k = *a;
+    if (k.mult == 0.f) k.mult = 1.f;
     if (v->dtype == PICOLM_F32)
-        branch_norm_kernel<float><<<v->rows, threads, 0, v->stream>>>((float*)v->out, (const float*)v->in, (float*)v->extra[0], *a);
+        branch_norm_kernel<float><<<v->rows, threads, 0, v->stream>>>((float*)v->out, (const float*)v->in, (float*)v->extra[0], k);
     else
-        branch_norm_kernel<bf16_t><<<v->rows, threads, 0, v->stream>>>((float*)v->out, (const float*)v->in, (bf16_t*)v->extra[0], *a);
+        branch_norm_kernel<bf16_t><<<v->rows, threads, 0, v->stream>>>((float*)v->out, (const float*)v->in, (bf16_t*)v->extra[0], k);
     PICOLM_LAUNCH_CHECK("branch_norm");
     return 0;
 }
@@ -589,7 +595,7 @@ extern "C" int picolm_call_layer_norm(void* user, const picolm_step_view* v) {
 // ---- rotation of stretches of a row by the token's position ---------------------------------------------
 // A thread a pair (or an entry that is only copied); a workgroup a row.  The stretches of the second group follow
 // those of the first in the threads' order; the normed stretch comes last and takes the whole workgroup's sum.
-__global__ __launch_bounds__(256) void rotate_heads_kernel(picolm_rotate_heads_args a, const float* __restrict__ in, float* __restrict__ out,
+__global__ __launch_bounds__(256) void rotate_heads_kernel(picolm_rotate_heads_args a, const float* in, float* out,       // (may be one buffer)
                                                            const int32_t* __restrict__ tok_pos) {
     __shared__ float scratch[16];
     const size_t row = blockIdx.x;

@@ -168,15 +168,20 @@ class ProgramBuilder:
         self.ops.append(Op(kind=OP_RMSNORM, rows=rows, inp=x, out=out, weight=self._ptr(norm.weight), k=norm.weight.shape[0],
                            eps=norm.eps))
 
-    def note_norm(self, x: int, norm: NormRef, buffer: int) -> None:
-        """The operation just appended has also left the RMSNorm `norm` of the rows in buffer `x` in
-        `buffer`: a part that asks for that norm next, with nothing in between, takes it from there."""
-        self._written_norm = (len(self.ops), x, norm.weight.data_ptr(), norm.eps, buffer)
+    def note_norm(self, x: int, norm: NormRef | None, buffer: int) -> None:
+        """The operation just appended has also left the RMSNorm `norm` of the rows in buffer `x` (None:
+        those rows themselves, in the dtype that products read) in `buffer`: a part that asks for it
+        next, with nothing in between, takes it from there."""
+        self._written_norm = (len(self.ops), x, *self._norm_key(norm), buffer)
 
-    def written_norm(self, x: int, norm: NormRef) -> int | None:
-        if self._written_norm is not None and self._written_norm[:4] == (len(self.ops), x, norm.weight.data_ptr(), norm.eps):
+    def written_norm(self, x: int, norm: NormRef | None) -> int | None:
+        if self._written_norm is not None and self._written_norm[:4] == (len(self.ops), x, *self._norm_key(norm)):
             return self._written_norm[4]
         return None
+
+    @staticmethod
+    def _norm_key(norm: NormRef | None) -> tuple:
+        return (norm.weight.data_ptr(), norm.eps) if norm is not None else (0, 0.0)
 
     def materialize(self, src: Rows, rows: int = ROWS_STEP) -> int:
         """The buffer that holds `src`'s rows, after running the norm they are the result of, if any,

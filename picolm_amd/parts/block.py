@@ -42,6 +42,15 @@ class PreNormBlock(Block):
         self.ffn.emit(b, self.ffn_norm.emit(b, x), x, after, after_when)
 
 
+def _plain_rows(b, x: int, width: int, name: str) -> int:
+    """The float rows in buffer `x` in the dtype that products read, in the buffer `name`."""
+    from ..engine.program import _DT, F32
+    from .calls import GATE_NONE, GateRowsArgs, emit_library_call
+    plain = b.buffer(name, width, b.dtype)
+    emit_library_call(b, "gate_rows", GateRowsArgs(width, GATE_NONE, width, 0, F32, 0, 0, _DT[b.dtype], None), plain, inp=x)
+    return plain
+
+
 class _NoMixer(Mixer):
     """The mixer of a block that has none: it asks nothing of the cache."""
 
@@ -184,15 +193,6 @@ class PostNormBlock(Block):
         emit_library_call(b, "gated_postnorm", GatedPostnormArgs(b._ptr(ref.weight), b._ptr(bias), self.D, self.alpha, ref.eps), x,
                           inp=branch, extra=extra)
 
-    def _plain_rows(self, b, x: int) -> int:
-        """The residual rows in the dtype that products read."""
-        import torch
-        from ..engine.program import _DT, F32
-        from .calls import GATE_NONE, GateRowsArgs, emit_library_call
-        plain = b.buffer("postnorm.plain", self.D, b.dtype)
-        emit_library_call(b, "gate_rows", GateRowsArgs(self.D, GATE_NONE, self.D, 0, F32, 0, 0, _DT[b.dtype], None), plain, inp=x)
-        return plain
-
     def emit(self, b, x: int, after=None, after_when: int = 0) -> None:
         import torch
         from ..engine.program import Rows
@@ -206,7 +206,7 @@ class PostNormBlock(Block):
             emit_library_call(b, "token_shift", TokenShiftArgs(b._ptr(self.mu), D, 0), reads, inp=x, extra=[plain] if self.gates else [],
                               uses_state=True)
         else:
-            plain = reads = self._plain_rows(b, x)
+            plain = reads = _plain_rows(b, x, self.D, "postnorm.plain")
         branch = b.buffer("postnorm.branch", D, torch.float32)
         self.inner.emit(b, Rows(reads), branch, accumulate=False)
         self._join(b, x, branch, plain, 0, self.mixer_norm, leaves_plain=self.ffn is not None)
@@ -258,6 +258,63 @@ class SandwichBlock(Block):
         if self.ffn is not None:
             self.ffn.emit(b, self.ffn_norm.emit(b, x), branch, accumulate=False)
             self._join(b, x, branch, None, self.ffn_after, following)
+
+
+class OutputNormBlock(Block):
+    """A norm behind each sublayer and none ahead of it:
+        x <- x + mult norm1(mixer(x));   x <- x + mult norm2(ffn(x))
+    A block without a feed-forward has the first half only.  The sublayers read the residual rows
+    themselves; where products read another dtype than the rows have, the operation that adds a branch
+    leaves the new rows in it too (or the norm that meets them, if the next block has one on entry)."""
+    graph_safe = True      # launches depend on device memory only
+
+    def __init__(self, mixer: Mixer, mixer_after: Norm, ffn: FeedForward | None, ffn_after: Norm | None, mult: float = 1.0):
+        if (ffn is None) != (ffn_after is None):
+            raise ValueError("a feed-forward and its norm come together")
+        if not mult:
+            raise ValueError("a factor of nought on the branches")
+        self.mixer, self.mixer_after, self.ffn, self.ffn_after, self.mult = mixer, mixer_after, ffn, ffn_after, float(mult)
+
+    def children(self):
+        return [p for p in (self.mixer, self.mixer_after, self.ffn, self.ffn_after) if p is not None]
+
+    def _reads(self, b, x: int):
+        """The residual rows as a sublayer's input."""
+        import torch
+        from ..engine.program import Rows
+        if b.dtype == torch.float32:
+            return Rows(x)
+        written = b.written_norm(x, None)
+        return Rows(_plain_rows(b, x, self.mixer_after.size, "norm.out") if written is None else written)
+
+    def _join(self, b, x: int, branch: int, bias, norm, following, plain: bool) -> None:
+        """x <- x + mult norm(branch + bias), and the norm `following` of the new x where it is given, or
+        with `plain` the new x in the dtype that products read."""
+        import torch
+        from .calls import BranchNormArgs, emit_library_call
+        ref = norm_ref_of(norm)
+        if ref is None:
+            raise ValueError("a block with norms behind its sublayers takes RMS norms there")
+        plain = plain and following is None and b.dtype != torch.float32
+        extra = [b.buffer("norm.out", norm.size, b.dtype)] if following is not None or plain else []
+        emit_library_call(b, "branch_norm", BranchNormArgs(b._ptr(bias), b._ptr(ref.weight), b._ptr(following.weight if following else None),
+                                                           norm.size, ref.eps, following.eps if following else 0.0, self.mult, int(plain)),
+                          x, inp=branch, extra=extra)
+        if extra:
+            b.note_norm(x, following, extra[0])
+
+    def emit(self, b, x: int, after=None, after_when: int = 0) -> None:
+        import torch
+        # after_when = 1: the final norm follows, of which the head takes the rows it wants
+        following, plain = (after, after is None) if after_when == 0 else (None, False)
+        branch = b.buffer("branch.out", self.mixer_after.size, torch.float32)
+        bias = self.mixer.emit_branch(b, self._reads(b, x), branch)
+        if self.ffn is None:
+            self._join(b, x, branch, bias, self.mixer_after, following, plain)
+            return
+        self._join(b, x, branch, bias, self.mixer_after, None, True)
+        self.ffn.emit(b, self._reads(b, x), branch, accumulate=False)
+        self._join(b, x, branch, None, self.ffn_after, following, plain)
 
 
 class LoopSum(Block):

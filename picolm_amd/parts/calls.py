@@ -3,7 +3,7 @@ the engine hands the running step to, with a structure of sizes, offsets, consta
 pointers.  The structures here mirror that header field by field."""
 from __future__ import annotations
 
-from ctypes import Structure, c_float, c_int32, c_int64, c_void_p
+from ctypes import Structure, c_double, c_float, c_int32, c_int64, c_void_p
 
 from .. import kernels
 
@@ -20,7 +20,7 @@ class SinkAttentionArgs(Structure):
                 ("chunk", c_int32), ("maps", c_int32), ("out_float", c_int32), ("unit_qk", c_int32), ("in_bias", c_void_p),
                 ("cos_table", c_void_p), ("sin_table", c_void_p), ("table_positions", c_int32), ("rot_dims", c_int32), ("rot_half", c_int32),
                 ("norm_all", c_int32), ("keep_first", c_int32), ("softcap", c_float), ("gate_per_head", c_int32), ("first_col", c_int32),
-                ("out_stride", c_int32), ("out_off", c_int32), ("out_mult", c_float)]
+                ("out_stride", c_int32), ("out_off", c_int32), ("out_mult", c_float), ("temp_coef", c_float), ("temp_every", c_double)]
 
 
 class ShortConvArgs(Structure):
@@ -99,7 +99,8 @@ class ChannelDecaysArgs(Structure):
 
 
 class BranchNormArgs(Structure):
-    _fields_ = [("bias", c_void_p), ("weight", c_void_p), ("next_weight", c_void_p), ("width", c_int32), ("eps", c_float), ("next_eps", c_float)]
+    _fields_ = [("bias", c_void_p), ("weight", c_void_p), ("next_weight", c_void_p), ("width", c_int32), ("eps", c_float), ("next_eps", c_float),
+                ("mult", c_float), ("plain", c_int32)]
 
 
 class RouteTopArgs(Structure):
@@ -140,14 +141,15 @@ class MapDifferenceArgs(Structure):
 
 
 class LinearAttentionArgs(Structure):
-    _fields_ = [("decays", ChannelDecaysArgs), ("scan", DecayScanArgs), ("norm", GatedNormArgs)]
+    _fields_ = [("decays", ChannelDecaysArgs), ("scan", DecayScanArgs), ("norm", GatedNormArgs), ("cos_table", c_void_p), ("sin_table", c_void_p),
+                ("table_positions", c_int32), ("rot_dims", c_int32), ("rot_half", c_int32)]
 
 
 GATE_NONE, GATE_SILU, GATE_SIGMOID = 0, 1, 2
 DECAY_PER_ROW, DECAY_EXPONENTIAL, DECAY_FIXED = 1, 2, 3
 DECAY_SCAN_MAX_KEY_DIM = 256
 MAP_RELU_SQUARED, MAP_SOFTCAP, MAP_SCALE = 1, 2, 3
-SCORE_PICKED_SOFTMAX, SCORE_SOFTMAX_ALL, SCORE_SIGMOID = 0, 1, 2
+SCORE_PICKED_SOFTMAX, SCORE_SOFTMAX_ALL, SCORE_SIGMOID, SCORE_SOFTMAX_KEPT = 0, 1, 2, 3
 EXPERT_SILU_GATED, EXPERT_CLAMPED = 0, 1
 RULE_OUTER_PRODUCT, RULE_DELTA = 0, 1
 STATE_SCAN_MAX_KEY_DIM = 256

@@ -78,6 +78,7 @@ class RoutedExperts(FeedForward):
     scoring "picked_softmax": the largest z + b are picked (ties: the lower index) and w is the
     softmax over the picked z + b alone.  scoring "softmax_all": s = softmax(z) over every router
     output, the largest s + b are picked, and w = s_k / (sum of the picked s + 1e-20) * weight_scale.
+    scoring "softmax_kept": the same picks, w = s_k * weight_scale.
     expert(h) = down(silu(gate h) * (up h)), no biases; the last `identity` router outputs have no
     tensors and stand for experts that give h back; `shared_size` > 0 adds one more expert of that
     inner width that every row passes, multiplied by sigmoid(w_sg . h), one number a row, where
@@ -85,7 +86,7 @@ class RoutedExperts(FeedForward):
     output.  The router's logits, the picks and their weights are float; only the picked experts'
     weights are read."""
     graph_safe = True      # launches depend on device memory only
-    SCORINGS = {"picked_softmax": 0, "softmax_all": 1, "sigmoid": 2}
+    SCORINGS = {"picked_softmax": 0, "softmax_all": 1, "sigmoid": 2, "softmax_kept": 3}
     ACTIVATIONS = {"silu_gated": 0, "clamped": 1}
 
     def __init__(self, prefix: str, hidden_size: int, n_experts: int, top: int, expert_size: int, shared_size: int = 0,

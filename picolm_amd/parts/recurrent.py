@@ -299,13 +299,14 @@ class LinearAttention(Mixer):
 
     def __init__(self, prefix: str, hidden_size: int, n_heads: int, key_dim: int, value_dim: int, eps: float, decay=None, tau: float | None = None,
                  rank: int | None = None, silu_qkv: bool = False, q_scale: float = 1.0, k_scale: float = 1.0, norm: str = "head",
-                 norm_weight: bool = True, gate: str = "silu"):
+                 norm_weight: bool = True, gate: str = "silu", position=None):
         """`decay`: a factor per head.  Without it the decays are the token's own, per head and key
         channel, through the tensors a1, a2 and a2.b and the exponent 1/`tau`; `rank`: rows of a1
         (None: as many as the checkpoint's tensor has).  `silu_qkv`: q, k and v pass a silu.  `norm`:
         "head" norms every head's output by itself, "all" the heads together; `norm_weight`: with the
         tensor `norm`, of the size that is normed.  `gate`: the function of W_g h that multiplies the
-        normed outputs."""
+        normed outputs.  `position`: a `RotaryEmbedding` over the first entries of every head of q and k
+        (as many as it was made for), ahead of the factors."""
         if not 1 <= key_dim <= DECAY_SCAN_MAX_KEY_DIM:
             raise ValueError(f"a state with keys of {key_dim}: the kernel takes 1 to {DECAY_SCAN_MAX_KEY_DIM}")
         if (decay is None) == (tau is None):
@@ -322,6 +323,9 @@ class LinearAttention(Mixer):
         self.silu_qkv, self.q_scale, self.k_scale = bool(silu_qkv), float(q_scale), float(k_scale)
         self.norm_group = value_dim if norm == "head" else n_heads * value_dim
         self.has_norm_weight, self.gate = bool(norm_weight), gate
+        if position is not None and (silu_qkv or not 0 < position.head_dim <= key_dim):
+            raise ValueError(f"a rotation of {position.head_dim} entries of a head of {key_dim} (which takes no silu)")
+        self.position = position
         self.state_base = 0
         self.gives_products = False        # True: a part around this one runs proj and o
         qk, vv = n_heads * key_dim, n_heads * value_dim
@@ -334,7 +338,11 @@ class LinearAttention(Mixer):
         self.decay = self.a2 = self.a2_bias = self.norm = None
 
     def children(self):
-        return [] if self.gives_products else [self.proj, self.o]
+        return ([] if self.gives_products else [self.proj, self.o]) + ([self.position] if self.position is not None else [])
+
+    def prepare(self, runtime: Runtime, max_positions: int) -> None:
+        if self.position is not None:
+            self.position.prepare(runtime, max_positions)
 
     def tensor_specs(self):
         p, qk = self.prefix, self.H * self.dk
@@ -390,4 +398,10 @@ class LinearAttention(Mixer):
             extra.append(b.buffer("scan.decays", qk, torch.float32))
         args.norm = GatedNormArgs(b._ptr(self.norm), self.norm_group, vv, self.norm_group, self.eps, 0, stride, at + 2 * qk + vv,
                                   self.GATES[self.gate], out_stride, out_off, mult)
+        if self.position is not None:
+            cos, sin, style = self.position.rotary_tables()
+            if cos is None:
+                raise ValueError(f"the rotation of {self.prefix} has no tables laid out (prepare)")
+            args.cos_table, args.sin_table, args.table_positions = b._ptr(cos), b._ptr(sin), cos.shape[0]
+            args.rot_dims, args.rot_half = self.position.head_dim, style
         emit_library_call(b, "linear_attention", args, out, inp=rows, extra=extra, uses_state=True)

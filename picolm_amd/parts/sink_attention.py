@@ -3,9 +3,11 @@ rotation of part of every head, an RMS norm of queries and keys per head (with a
 root mean square without one), a learned bias by distance, one more term in the softmax's
 denominator (a sink, learned per head or a constant), values of a size of their own or the keys
 themselves as values, stretches of positions or a window that bound what a query sees, first tokens that
-it sees beside its window, a cap on the scores, and a gate on the heads before the output projection.
+it sees beside its window, a cap on the scores, queries that grow with the position, keys and values of
+another layer, and a gate on the heads before the output projection.
 
     q, k, v, g = W h (+ b);  q, k <- turned by the position;  q <- rms(q) w_q,  k <- rms(k) w_k     per head
+    q <- q (1 + coef ln(floor((p + 1) / every) + 1))                   p: the token's position
     s_ij = scale (q_i . k_j) + rel[bucket(i - j)][head]                j <= i, and floor(i / chunk) = floor(j / chunk)
     p_ij = exp(s_ij) / (exp(sink_head) + sum_j' exp(s_ij'))            the sink is a term of the denominator only
     out  = W_o (concat_heads(sum_j p_ij v_j) * sigmoid(g)) (+ b_o)     g: a number an entry, or one a head
@@ -56,7 +58,7 @@ class SinkAttention(Mixer):
                  qk_norm: bool = True, sink: bool = True, gate: bool = True, proj_bias: bool = False, position=None,
                  unit_qk: bool = False, fixed_sink: float | None = None, chunk: int = 0, values_are_keys: bool = False,
                  norm_all: bool = False, softcap: float = 0.0, window: int = 0, keep_first: int = 0, gate_per_head: bool = False,
-                 out_bias: bool = False):
+                 out_bias: bool = False, q_temp: tuple | None = None, reads_keys: bool = False):
         """`has_bias`: scores get the bias by distance, from a table of `bias_rows` rows (None: as many
         as the checkpoint's tensor has) that reaches to `bias_max`.  `proj_bias`: q, k and v have
         biases, the tensors `<name>.b`.  `position`: a `RotaryEmbedding` over the first entries of
@@ -68,7 +70,10 @@ class SinkAttention(Mixer):
         key as projected, before rotation and norm.  `norm_all`: the norm of q and the norm of k each
         cover all heads (weights of the projection's size).  `window`, `keep_first`: what a query sees
         (0: every key); the cache keeps all keys and a decode step visits those that are seen.
-        `out_bias`: the output projection has one, the tensor `o.b`."""
+        `out_bias`: the output projection has one, the tensor `o.b`.  `q_temp` = (coef, every): the
+        factor on the queries (after everything else that makes them).  `reads_keys`: the layer has no
+        keys and values of its own and reads the cache entry of another layer call, which keeps the
+        same kind of them."""
         if n_heads % n_kv_heads:
             raise ValueError(f"{n_heads} heads do not split over {n_kv_heads} KV heads")
         self.prefix, self.D = prefix, hidden_size
@@ -96,9 +101,13 @@ class SinkAttention(Mixer):
             raise ValueError("a cap on the scores and a bias by distance do not go together")
         self.norm_all, self.softcap, self.window, self.keep_first = bool(norm_all), float(softcap), int(window), int(keep_first)
         self.gate_per_head, self.has_out_bias = bool(gate_per_head) and gate, bool(out_bias)
-        names = [prefix + "q", prefix + "k"] + ([] if values_are_keys else [prefix + "v"]) + ([prefix + "g"] if gate else [])
-        sizes = ([n_heads * head_dim, n_kv_heads * head_dim] + ([] if values_are_keys else [n_kv_heads * v_head_dim]) +
-                 ([n_heads if gate_per_head else n_heads * v_head_dim] if gate else []))
+        if q_temp is not None and not q_temp[1] > 0:
+            raise ValueError(f"queries that grow every {q_temp[1]} positions")
+        self.q_temp, self.reads_keys = None if q_temp is None else (float(q_temp[0]), float(q_temp[1])), bool(reads_keys)
+        own = [] if reads_keys else [("k", n_kv_heads * head_dim)] + ([] if values_are_keys else [("v", n_kv_heads * v_head_dim)])
+        self.biased = 1 + len(own)         # matrices of the stacked product that may have a bias
+        stacked = [("q", n_heads * head_dim)] + own + ([("g", n_heads if gate_per_head else n_heads * v_head_dim)] if gate else [])
+        names, sizes = [prefix + n for n, _ in stacked], [size for _, size in stacked]
         self.proj = Linear(names, sizes, hidden_size)
         self.o = Linear([prefix + "o"], [hidden_size], n_heads * v_head_dim)
         self.q_norm = self.k_norm = self.bias = self.sink = self.in_bias = self.o_bias = None
@@ -115,14 +124,15 @@ class SinkAttention(Mixer):
         specs = []
         if self.qk_norm:
             over_q, over_k = (self.H, self.G) if self.norm_all else (1, 1)
-            specs += [TensorSpec(self.prefix + "q.norm", (over_q * self.d,), init="ones"),
-                      TensorSpec(self.prefix + "k.norm", (over_k * self.d,), init="ones")]
+            specs.append(TensorSpec(self.prefix + "q.norm", (over_q * self.d,), init="ones"))
+            if not self.reads_keys:
+                specs.append(TensorSpec(self.prefix + "k.norm", (over_k * self.d,), init="ones"))
         if self.has_bias:       # (-1: any number of rows; random weights need the number)
             specs.append(TensorSpec(self.prefix + "rel", (self.bias_rows if self.bias_rows is not None else -1, self.H)))
         if self.has_sink:
             specs.append(TensorSpec(self.prefix + "sink", (self.H,)))
         if self.proj_bias:
-            specs += [TensorSpec(n + ".b", (size,)) for n, size in zip(self.proj.names[:2 if self.values_are_keys else 3], self.proj.out_sizes)]
+            specs += [TensorSpec(n + ".b", (size,)) for n, size in zip(self.proj.names[:self.biased], self.proj.out_sizes)]
         if self.has_out_bias:
             specs.append(TensorSpec(self.prefix + "o.b", (self.D,)))
         return specs
@@ -130,7 +140,8 @@ class SinkAttention(Mixer):
     def load(self, fetch, runtime: Runtime) -> None:
         f32 = lambda name: fetch.get(self.prefix + name).to(torch.float32).contiguous()
         if self.qk_norm:
-            self.q_norm, self.k_norm = f32("q.norm"), f32("k.norm")
+            self.q_norm = f32("q.norm")
+            self.k_norm = None if self.reads_keys else f32("k.norm")
         if self.has_bias:
             rel = f32("rel")
             rows = distance_rows(rel.shape[0], self.bias_max)
@@ -142,7 +153,7 @@ class SinkAttention(Mixer):
         if self.has_out_bias:
             self.o_bias = f32("o.b")
         if self.proj_bias:          # one entry per column of the stacked product; the gate's columns get none
-            parts = [fetch.get(n + ".b").to(torch.float32) for n in self.proj.names[:2 if self.values_are_keys else 3]]
+            parts = [fetch.get(n + ".b").to(torch.float32) for n in self.proj.names[:self.biased]]
             parts.append(torch.zeros(self.proj.out_size - sum(p.numel() for p in parts), dtype=torch.float32, device=parts[0].device))
             self.in_bias = torch.cat(parts).contiguous()
 
@@ -180,15 +191,19 @@ class SinkAttention(Mixer):
         H, G, d, dv = self.H, self.G, self.d, self.dv
         width = stride
         q = b.buffer("sink_attn.q", H * d, b.dtype)
+        if b.binding is not None and bool(b.binding.writes) == self.reads_keys:
+            raise ValueError(f"{self.prefix}: a layer with keys of its own writes its cache entry, one that reads another's does not")
         q_off, k_off = 0, H * d
         v_off = k_off if self.values_are_keys else k_off + G * d
-        gate_off = (k_off + G * d if self.values_are_keys else v_off + G * dv) if self.has_gate else -1
+        gate_off = sum(self.proj.out_sizes[:self.biased]) if self.has_gate else -1
         args = SinkAttentionArgs(H, G, d, dv, width, q_off, k_off, v_off, gate_off, self.scale, self.eps,
                                  b._ptr(self.q_norm), b._ptr(self.k_norm), b._ptr(self.bias),
                                  0 if self.bias is None else self.bias.shape[1], b._ptr(self.sink))
         args.chunk, args.unit_qk, args.in_bias = self.chunk, int(self.unit_qk), b._ptr(self.in_bias)
         args.norm_all, args.softcap, args.keep_first, args.gate_per_head = int(self.norm_all), self.softcap, self.keep_first, int(self.gate_per_head)
         args.first_col, args.out_stride, args.out_off, args.out_mult = first_col, out_stride, out_off, mult
+        if self.q_temp is not None:
+            args.temp_coef, args.temp_every = self.q_temp
         if self.position is not None:
             cos, sin, style = self.position.rotary_tables()
             if cos is None:
