@@ -141,8 +141,12 @@ def gated(h, W, p):
     return (silu(h @ W[p + "gate"].T) * (h @ W[p + "up"].T)) @ W[p + "down"].T
 
 
+def router_logits(h, W, p):
+    return h @ W[p + "router"].T
+
+
 def router_scores(h, W, p):
-    z = h @ W[p + "router"].T
+    z = router_logits(h, W, p)
     e = np.exp(z - z.max(axis=1, keepdims=True))
     return e / e.sum(axis=1, keepdims=True)
 
@@ -158,9 +162,9 @@ def routed_experts(h, W, p, mlp):
 
 
 def router_margins(h, W, p, mlp):
-    """Per row, how far the last picked score lies above the first one not picked."""
-    top, s = mlp["router"]["top"], -np.sort(-router_scores(h, W, p), axis=1)
-    return s[:, top - 1] - s[:, top] if top < s.shape[1] else np.full(len(h), np.inf)
+    """Per row, how far the last pick's logit lies above the first one not picked."""
+    top, z = mlp["router"]["top"], -np.sort(-router_logits(h, W, p), axis=1)
+    return z[:, top - 1] - z[:, top] if top < z.shape[1] else np.full(len(h), np.inf)
 
 
 def feed_forward(h, W, p, mlp):
