@@ -358,7 +358,58 @@ def _zalalix_rooflines(cfg: dict, T: int, n_seq: int, context: int) -> dict:
     return {"prefill": pre, "decode": dec}
 
 
+def _belorax_trio(width: int, heads: int, kv_rank: int, rot_dim: int, experts: int, top: int, vocab: int, zalalix: tuple):
+    """A Belorax of four layers (retention; attention; latent attention; attention that reads the second
+    layer's keys) with heads of 128 (in the latent layer with `rot_dim` of them turned, over latents of
+    `kv_rank`), a KV head for four query heads, and `experts` experts as wide as the model of which a
+    token uses `top` in every layer.  The Satedra of as many layers of the same width, heads, vocabulary
+    and experts (no identity picks, no shared expert) whose windows show every key: the closest model for
+    the attention and the experts.  And a Zalalix of the same width and heads, whose second pair of
+    layers holds a retention: the closest one for the states."""
+    mlp = dict(kind="moe", router=dict(experts=experts, top=top), expert=dict(ff=width))
+    attn = dict(heads=heads, kv_heads=max(heads // 4, 1), dim=128, vdim=128, scale=128 ** -0.5, q_temp=dict(coef=0.1, every=4096))
+    mixers = [("retention", dict(heads=heads, dim=128, vdim=128, decay=[1.0 - 2.0 ** -(5.0 + 5.0 * i / heads) for i in range(heads)],
+                                 rot=dict(base=10000.0, dims=128))),
+              ("attention", attn),
+              ("latent_attention", dict(heads=heads, dim=128 - rot_dim, rot_dim=rot_dim, vdim=128, kv_rank=kv_rank, scale=128 ** -0.5,
+                                        rot=dict(base=10000.0, dims=rot_dim, scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0)))),
+              ("attention", dict(attn, kv_from=1))]
+    bel = dict(architecture="Belorax", vocab=vocab, width=width, embedding=dict(scale=width ** 0.5), residual_mult=0.5, norm=dict(eps=1e-5),
+               layers=[dict(type=t, mixer=m, mlp=mlp) for t, m in mixers])
+    sat, _ = _satedra_pair(width, heads, kv_rank, rot_dim, 1 << 20, experts, top, vocab, len(mixers))
+    for layer in sat["layers"]:
+        layer["mlp"] = dict(layer["mlp"], router=dict(experts=experts, top=top, identity=0, scale=1.0), shared=None)
+    return bel, sat, _zalalix_pair(*zalalix)[0]
+
+
+def _belorax_rooflines(cfg: dict, T: int, n_seq: int, context: int) -> dict:
+    """As _satedra_rooflines and _zalalix_rooflines: the attention over every earlier key, the states and
+    the picked experts' products."""
+    mfma, valu, hbm = PEAK_TFLOPS["bf16"] * 1e12, PEAK_TFLOPS["fp32"] * 1e12, HBM_PEAK_GBS * 1e9
+    names = ("sink_attention", "linear_attention", "routed_experts")
+    pre, dec = {k: 0.0 for k in names}, {k: 0.0 for k in names}
+    D, seen = cfg["width"], T * (T + 1) / 2
+    for layer in cfg["layers"]:
+        m, mlp = layer["mixer"], layer.get("mlp")
+        if layer["type"] == "retention":
+            pre["linear_attention"] += 5.0 * T * m["heads"] * m["dim"] * m["vdim"] / valu
+            dec["linear_attention"] += n_seq * 2 * m["heads"] * m["dim"] * m["vdim"] * 4 / hbm
+        else:
+            latent = layer["type"] == "latent_attention"
+            key_and_value = 2 * m["kv_rank"] + m["rot_dim"] if latent else m["dim"] + m["vdim"]
+            pre["sink_attention"] += 2.0 * m["heads"] * key_and_value * seen / mfma
+            dec["sink_attention"] += n_seq * context * (1 if latent else m["kv_heads"]) * key_and_value * 2 / hbm
+        if mlp and mlp["kind"] == "moe":
+            E, top, F = mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"]
+            pre["routed_experts"] += 2.0 * 3 * T * top * D * F / mfma
+            dec["routed_experts"] += min(n_seq * top, E) * 3 * D * F * 2 / hbm
+    return {"prefill": pre, "decode": dec}
+
+
 DESIGN_SIZES = {
+    "belorax": [("width 1024", (1024, 8, 96, 32, 8, 2, 32000, (1024, 8, 2, 4096, 2752, 32000, 2, 768))),
+                ("width 2048", (2048, 16, 96, 32, 8, 2, 32000, (2048, 16, 4, 8192, 5504, 32000, 2, 768))),
+                ("width 4096", (4096, 32, 96, 32, 16, 2, 128256, (4096, 32, 8, 14336, 9600, 128256, 2, 768)))],
     "zalalix": [("width 1024", (1024, 8, 2, 4096, 2752, 32000, 2, 768)), ("width 2048", (2048, 16, 4, 8192, 5504, 32000, 2, 768)),
                 ("width 4096", (4096, 32, 8, 14336, 9600, 128256, 1, 768))],
     "kekelix": [("width 1024", (1024, 8, 1536, 8, 2, 32000, 4)), ("width 2048", (2048, 16, 1536, 8, 2, 32000, 4)),
@@ -406,7 +457,8 @@ def _zarinex_rooflines(cfg: dict, T: int, n_seq: int, context: int) -> dict:
 def design_comparison(design: str, T: int, n_seq: int, context: int, steps: int) -> dict:
     """Prefill and decode throughput of `design` at a few sizes that resemble real layers (random
     weights), beside the closest model the library has at equal size (for Begopel the Llama, for
-    Zarinex the Begopel, for Satedra the Zarinex, for Kekelix the Satedra, for Zalalix the Begopel), and the GPU time of one prefill step and one decode step by operation."""
+    Zarinex the Begopel, for Satedra the Zarinex, for Kekelix the Satedra, for Zalalix the Begopel,
+    for Belorax the Satedra and the Zalalix), and the GPU time of one prefill step and one decode step by operation."""
     import torch
 
     from picolm_amd.config import LlamaConfig, resolve
@@ -466,6 +518,14 @@ def design_comparison(design: str, T: int, n_seq: int, context: int, steps: int)
 
     for name, size in DESIGN_SIZES[design]:
         print(f"[bench] {design} {name}", file=sys.stderr, flush=True)
+        if design == "belorax":
+            bel, sat, zal = _belorax_trio(*size)
+            res = {n: measure(resolve(c).parse_config(c), c["vocab"]) for n, c in ((design, bel), ("satedra", sat), ("zalalix", zal))}
+            out["sizes"].append({"size": name, "layer_runs": len(bel["layers"]), **res,
+                                 "fraction_of_roofline": fractions_of(_belorax_rooflines(bel, T, n_seq, context), res[design]),
+                                 "satedra_fraction_of_roofline": fractions_of(_satedra_rooflines(sat, T, n_seq, context), res["satedra"]),
+                                 "zalalix_fraction_of_roofline": fractions_of(_zalalix_rooflines(zal, T, n_seq, context), res["zalalix"])})
+            continue
         if design == "zalalix":
             zal, beg = _zalalix_pair(*size)
             a = measure(resolve(zal).parse_config(zal), zal["vocab"])
